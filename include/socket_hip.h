@@ -32,7 +32,7 @@
 extern "C" {
 #endif
 
-#define SOCKET_ABI_VERSION 4   /* 4: the packed scorers take a flags word */
+#define SOCKET_ABI_VERSION 5   /* 5: the structs of the row, attention and recurrence kernels grew */
 
 /* status codes */
 #define SOCKET_OK 0
@@ -486,14 +486,28 @@ int socket_block_sparse_attention(const void* q, const void* k, const void* v, i
  * in libsocket_core.so, which libsocket_hip.so depends on.
  * ---------------------------------------------------------------------- */
 
+/* Average over depth: a layer's result x' is stored at `result`, and what goes on is
+ *   sum over j < n of w[j] * past[j * past_stride + i] + w[n] * x'[i]
+ * past: the n earlier results (the embedding output first), each [rows, dim] fp32; w fp32
+ * [n + 1] on the device; w NULL: no averaging.  `result` overlaps none of the n. */
+typedef struct socket_depth_mix {
+  const float* past;
+  int64_t past_stride;
+  const float* w;
+  int n;
+  float* result;
+} socket_depth_mix;
+
 /* The step between two sublayers, per row of `dim` elements:
  *   y = scale_a * a + scale_b * b          pending sublayer output (b may be NULL)
- *   x_out = x + y * rsqrt(mean(y^2) + eps) * post_w     (post_w NULL: x + y)
+ *   x' = x + y * rsqrt(mean(y^2) + eps) * post_w     (post_w NULL: x + y)
+ *   x_out = x', or its average with earlier results (depth.w)
  *   h_out = x_out * rsqrt(mean(x_out^2) + eps) * pre_w
- * x, x_out fp32; with `a` NULL nothing is added.  x may be NULL: the row is then
- * looked up as embed[ids[row]] (embed of `dtype`, ids int32 or int64, clamped to
- * the table).  x_out may be NULL or equal to x.  a / b are of `dtype`, or fp32
- * with pending_f32; h_out (may be NULL) is of `dtype`; norm weights are fp32. */
+ * x, x_out fp32, rows of x `x_stride` elements apart (0: dim); with `a` NULL nothing is
+ * added.  x may be NULL: the row is then looked up as embed[ids[row]] * embed_scale (embed
+ * of `dtype`, ids int32 or int64, clamped to the table).  x_out may be NULL or equal to x.
+ * a / b are of `dtype`, or fp32 with pending_f32; h_out (may be NULL) is of `dtype`; norm
+ * weights are fp32. */
 typedef struct socket_residual {
   const float* x;
   const void* embed;
@@ -511,15 +525,21 @@ typedef struct socket_residual {
   int dim;
   float* x_out;
   void* h_out;
+  float embed_scale;
+  int64_t x_stride;
+  socket_depth_mix depth;
 } socket_residual;
 int socket_residual_norm(const socket_residual* args, int64_t rows, void* stream);
 
 /* Matrix-vector products of a decode step, bf16 weights [N,K] row-major, M <= 4
  * rows, fp32 accumulation.  kind 0: y = s1 * (x1 . w1[n]) (+ s2 * (x2 . w2[n]) when
- * x2 is given).  kind 1: clamped gated unit of g = x1 . w1[n], u = x1 . w2[n] (see
- * socket_clamped_glu).  With `norm` the row x1 is the h of socket_residual_norm,
- * worked out by every workgroup for itself (x_out is written once and must not
- * alias x); K1 = norm->dim then.  K1 and K2 multiples of 8; y bf16 or fp32.
+ * x2 is given) + b1[n].  kind 1 / 2: clamped / SiLU gated unit (see socket_gated_unit) of
+ * g = x1 . w1[n] + b1[n], u = x1 . w2[n] + b2[n].  Biases are bf16, NULL: none.  With
+ * `norm` the row x1 is the h of socket_residual_norm, worked out by every workgroup for
+ * itself (x_out is written once and must not alias x; no averaging over depth); K1 =
+ * norm->dim then.  With `res` (fp32 [M,N]; kind 0, one product, no norm) the residual sum
+ * rides along: x' = res + product, and y (fp32) is x' or, with depth.w, its average.
+ * K1 and K2 multiples of 8; y bf16 or fp32.
  * SOCKET_ERR_UNSUPPORTED for other shapes: the caller uses a library product. */
 typedef struct socket_rows_linear {
   const socket_residual* norm;
@@ -534,12 +554,17 @@ typedef struct socket_rows_linear {
   void* y;
   int y_f32;
   int M, N;
+  const void* b1;
+  const void* b2;
+  const float* res;
+  socket_depth_mix depth;
 } socket_rows_linear;
 int socket_rows_linear_bf16(const socket_rows_linear* args, void* stream);
 
-/* out[r, j] = g * sigmoid(1.702 g) * (u + 1), g = min(gu[r, j], limit),
- * u = clamp(gu[r, ff + j], -limit, limit); gu [rows, 2 ff], out [rows, ff]. */
-int socket_clamped_glu(const void* gu, void* out, int dtype, int64_t rows, int ff, float limit, void* stream);
+/* Gated unit of the halves of gu [rows, 2 ff], out [rows, ff].  kind 1 (clamped):
+ * out[r, j] = g * sigmoid(1.702 g) * (u + 1), g = min(gu[r, j], limit), u = clamp(gu[r, ff + j],
+ * -limit, limit).  kind 2 (SiLU): g * sigmoid(g) * u. */
+int socket_gated_unit(const void* gu, void* out, int dtype, int64_t rows, int ff, int kind, float limit, void* stream);
 
 /* Rotate-half rotary embedding of the q and k heads of a projected row: element i
  * < rot_dims / 2 of a head is paired with i + rot_dims / 2, the rest passes.
@@ -585,8 +610,13 @@ int socket_chunk_ring_store(const void* k, int64_t k_sb, int64_t k_st, int64_t k
  * Scores are (q . k) * scale, then softcap * tanh(score / softcap) when softcap > 0.
  * Keys at positions >= pos0 come from k_new / v_new (strides b, t, g), older ones of the
  * same chunk from slot j % chunk of the ring.  q [B,T,H,D] (strides b, t, h), out
- * [B,T,H,D] contiguous.  With pos (T = 1, device position) every key comes from the ring.
- * force_simple != 0 takes the lane-per-key kernel whatever the shape. */
+ * [B,T,H,Dv] contiguous.  With pos (T = 1, device position) every key comes from the ring.
+ * Dv: width of the values, at most D + D2 (0: D).  k_from: position of the first row of k_new / v_new
+ * (pos0 as above; 0: they hold every position).  k2 (may be NULL): D2 more key dimensions that
+ * all heads share, position j at row j (strides b, t); a query row then has D + D2 elements and
+ * a ring is not read (k_from 0, or pos with the ring holding D + D2 wide keys and no k2).
+ * gate (may be NULL; `dtype`, element h Dv + d of row (b, t)): the output is multiplied by its
+ * sigmoid.  force_simple != 0 takes the lane-per-key kernel whatever the shape. */
 typedef struct socket_chunk_attention {
   const void* q;
   int64_t q_stride_b, q_stride_t, q_stride_h;
@@ -605,13 +635,95 @@ typedef struct socket_chunk_attention {
   float scale, softcap;
   void* out;
   int force_simple;
+  int Dv;
+  int64_t k_from;
+  const void* k2;
+  int64_t k2_stride_b, k2_stride_t;
+  int D2;
+  const void* gate;
+  int64_t gate_stride_b, gate_stride_t;
 } socket_chunk_attention;
 int socket_chunk_attend(const socket_chunk_attention* args, void* stream);
+
+/* Latent attention: keys and values of all heads are products of one normalised latent row
+ * c [rank] per token, beside `rot` rotated key dimensions that all heads share.  The cache row
+ * of a position is [c, zeros up to rank_p, rotated part, zeros up to rank_p + rot_p] with rank_p
+ * and rot_p the sizes rounded up to 8.  Projected rows `in`: `in_dtype`, element strides b / t,
+ * columns cq_off (q_rank), c_off (rank), rot_off (rot).  Position of token t: *pos (T = 1) or
+ * pos0 + t; positions outside [0, n_pos) write nothing.
+ *
+ * socket_latent_rows: cache rows (c * rsqrt(mean(c^2) + eps) * c_norm; rotate-half of the rot
+ * columns) and, with cq_out [B,T,q_rank] (`dtype`), the normed query latent.
+ * socket_latent_absorb: q fp32 [B,T,H,dim + rot] (as projected) -> q_lat [B,T,H,rank_p + rot_p]
+ * (`dtype`): w_uk[h]^T q_h (w_uk [H dim, rank], `dtype`) and the rotated rest, zeros between;
+ * with `append` it also does what socket_latent_rows does for the cache.
+ * socket_rotate_tail: the last `rot` of the dim + rot elements of every head of q (`dtype`
+ * [B,T,H,dim + rot]) in place. */
+typedef struct socket_latent {
+  int dtype;
+  int B, T, H, dim, rot, q_rank, rank;
+  const void* in;
+  int in_f32;
+  int64_t in_stride_b, in_stride_t;
+  int cq_off, c_off, rot_off;
+  const float* q_norm;
+  const float* c_norm;
+  float eps;
+  const float* cos_sin;
+  int64_t n_pos;
+  int64_t pos0;
+  const int64_t* pos;
+  void* cache;
+  int64_t cache_stride_b, cache_stride_t;
+  void* cq_out;
+  int append;
+  const float* q;
+  const void* w_uk;
+  void* q_lat;
+} socket_latent;
+int socket_latent_rows(const socket_latent* args, void* stream);
+int socket_latent_absorb(const socket_latent* args, void* stream);
+int socket_rotate_tail(void* q, int dtype, int B, int T, int H, int dim, int rot, const float* cos_sin, int64_t n_pos,
+                       int64_t pos0, void* stream);
+
+/* Attention of q_lat (bf16) over the cache rows, values = their first `rank` elements, all heads
+ * of a token together: token (b, t) sees positions 0 .. (*pos or pos0) + t.  The keys are
+ * dealt to `splits` workgroups per (b, t, 16 heads); partial results: o [B*T, splits, H, rank_p]
+ * (weighted sums relative to the split's maximum), ml [B*T, splits, H, 2] (maximum in base-2
+ * units, sum of weights), fp32.  rank_p + rot_p <= 640, rank_p <= 512.
+ * socket_latent_values: merges `splits` partials (ml NULL: one, o already normalised) and gives
+ * out[b, t, h vdim + d] = (w_uv[h vdim + d] . o_h) * sigmoid(gate[b, t, h vdim + d]) (`dtype`;
+ * w_uv [H vdim, rank]; gate fp32 with gate_f32, NULL: none). */
+typedef struct socket_latent_attention {
+  int dtype;
+  int B, T, H, rank, rot, vdim;
+  const void* q_lat;
+  const void* cache;
+  int64_t cache_stride_b, cache_stride_t;
+  int64_t n_pos;
+  int64_t pos0;
+  const int64_t* pos;
+  float scale;
+  int splits;
+  float* o;
+  float* ml;
+  const void* w_uv;
+  const void* gate;
+  int gate_f32;
+  int64_t gate_stride_b, gate_stride_t;
+  void* out;
+} socket_latent_attention;
+int socket_latent_attend(const socket_latent_attention* args, void* stream);
+int socket_latent_values(const socket_latent_attention* args, void* stream);
 
 /* Gated linear recurrences with a decay per head and key channel and a state
  * S [dk, dv] per head, fp32 throughout:
  *   S <- g_t * S (rows);  delta rule: u = beta_t (v_t - S^T k_t), else u = v_t;
  *   S <- S + k_t u^T;  o_t = S^T q_t
+ * or, with rule 1 (generalized delta rule; dv any, H == Hk, no convolution, decay kind 2),
+ * with n_t = k_t / sqrt(sum k_t^2 + 1e-6) and removal rates a_t = sigmoid(column rate_off +
+ * h dk + c, + rate_bias) per key channel,
+ *   S <- g_t * S - (a_t * n_t) (S^T n_t)^T + k_t v_t^T   (both terms read the old S);  o_t = S^T q_t
  *   out_t = o_t * rsqrt(mean(o_t^2) + eps) * norm_w * gate_t
  * q, k (Hk heads), v (H heads) are columns of the projected rows `proj`; head h uses
  * q/k head h / (H / Hk).  taps >= 1: each channel of q | k | v first passes a causal
@@ -621,16 +733,19 @@ int socket_chunk_attend(const socket_chunk_attention* args, void* stream);
  * vectors, x / sqrt(sum x^2 + 1e-6); q is then multiplied by q_scale.
  * beta = sigmoid(column beta_off + h); beta_off < 0: no delta rule.
  * decay z = (decay_w [H dk, decay_rank] . columns decay_off ..) + decay_bias; kind 0:
- * log g = -exp(a_log[h]) * softplus(z); kind 1: log g = -softplus(-z) * inv_tau.
+ * log g = -exp(a_log[h]) * softplus(z); kind 1: log g = -softplus(-z) * inv_tau; kind 2:
+ * log g = -decay_rate * sigmoid(z).  decay_tanh: the low-rank product takes the tanh of its
+ * columns (rule 1, step; a scan is handed decay_z).
  * gate kind 0: sigmoid, 1: SiLU, of gate_w [H dv, gate_rank] . columns gate_off .., or of
  * column gate_off + h dv + c itself when gate_w is NULL.
+ * norm_w: [dv] shared by the heads, or with norm_per_head [H dv].
  * `fresh`: state and convolution inputs before pos0 are zero, whatever the buffers hold.
  *
  * socket_recurrence_step: one token per sequence, position *pos, out [B, H dv] (dtype).
  * socket_recurrence_scan: tokens t0 .. t0 + n - 1 of a portion of T tokens (rows t < 0 of
  * the portion are conv_state's); decay_z / gate_z hold the low-rank products of the
  * whole portion (decay_z fp32 or `dtype` [B,T,H dk], gate_z `dtype`); chunks of 64 (32
- * for dk > 128) tokens; workspace of socket_recurrence_workspace_bytes; o_buf fp32
+ * for dk > 128, with rule 1 for dk > 64) tokens; workspace of socket_recurrence_workspace_bytes; o_buf fp32
  * [B,n,H,dv] scratch; out [B,T,H dv].  socket_recurrence_conv_tail stores the last
  * taps - 1 inputs of the portion after its last scan. */
 typedef struct socket_recurrence {
@@ -667,10 +782,18 @@ typedef struct socket_recurrence {
   void* workspace;
   size_t workspace_bytes;
   void* out;
+  int rule;
+  int rate_off;
+  const float* rate_bias;
+  int decay_tanh;
+  float decay_rate;
+  int norm_per_head;
 } socket_recurrence;
+/* y[r, c] = tanh(x[r * x_stride + c]), y [rows, cols] contiguous, both of `dtype`. */
+int socket_tanh_rows(const void* x, int64_t x_stride, void* y, int dtype, int64_t rows, int cols, void* stream);
 int socket_recurrence_step(const socket_recurrence* args, void* stream);
-int socket_recurrence_chunk(int dk);
-size_t socket_recurrence_workspace_bytes(int B, int n, int H, int dk, int dv);
+int socket_recurrence_chunk(int dk, int rule);
+size_t socket_recurrence_workspace_bytes(int B, int n, int H, int dk, int dv, int rule);
 int socket_recurrence_scan(const socket_recurrence* args, void* stream);
 int socket_recurrence_conv_tail(const socket_recurrence* args, void* stream);
 

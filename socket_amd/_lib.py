@@ -35,17 +35,24 @@ _P, _I, _L, _Z = c_void_p, c_int, c_int64, c_size_t
 _F = c_float
 
 
+class DepthMix(ctypes.Structure):
+    """socket_depth_mix"""
+    _fields_ = [("past", _P), ("past_stride", _L), ("w", _P), ("n", _I), ("result", _P)]
+
+
 class Residual(ctypes.Structure):
     """socket_residual"""
     _fields_ = [("x", _P), ("embed", _P), ("ids", _P), ("ids64", _I), ("vocab", _I), ("a", _P), ("b", _P),
                 ("scale_a", _F), ("scale_b", _F), ("pending_f32", _I), ("post_w", _P), ("pre_w", _P), ("eps", _F),
-                ("dtype", _I), ("dim", _I), ("x_out", _P), ("h_out", _P)]
+                ("dtype", _I), ("dim", _I), ("x_out", _P), ("h_out", _P), ("embed_scale", _F), ("x_stride", _L),
+                ("depth", DepthMix)]
 
 
 class RowsLinear(ctypes.Structure):
     """socket_rows_linear"""
     _fields_ = [("norm", POINTER(Residual)), ("x1", _P), ("x2", _P), ("w1", _P), ("w2", _P), ("s1", _F), ("s2", _F),
-                ("K1", _I), ("K2", _I), ("kind", _I), ("limit", _F), ("y", _P), ("y_f32", _I), ("M", _I), ("N", _I)]
+                ("K1", _I), ("K2", _I), ("kind", _I), ("limit", _F), ("y", _P), ("y_f32", _I), ("M", _I), ("N", _I),
+                ("b1", _P), ("b2", _P), ("res", _P), ("depth", DepthMix)]
 
 
 class RopeHalf(ctypes.Structure):
@@ -64,7 +71,9 @@ class ChunkAttention(ctypes.Structure):
                 ("v_new", _P), ("v_stride_b", _L), ("v_stride_t", _L), ("v_stride_g", _L),
                 ("k_ring", _P), ("v_ring", _P), ("ring_stride_b", _L), ("ring_stride_g", _L), ("ring_stride_s", _L),
                 ("dtype", _I), ("B", _I), ("T", _I), ("H", _I), ("G", _I), ("D", _I), ("chunk", _I), ("pos0", _L),
-                ("pos", _P), ("scale", _F), ("softcap", _F), ("out", _P), ("force_simple", _I)]
+                ("pos", _P), ("scale", _F), ("softcap", _F), ("out", _P), ("force_simple", _I),
+                ("Dv", _I), ("k_from", _L), ("k2", _P), ("k2_stride_b", _L), ("k2_stride_t", _L), ("D2", _I),
+                ("gate", _P), ("gate_stride_b", _L), ("gate_stride_t", _L)]
 
 
 class Recurrence(ctypes.Structure):
@@ -77,7 +86,27 @@ class Recurrence(ctypes.Structure):
                 ("decay_w", _P), ("decay_rank", _I), ("decay_z", _P), ("decay_z_f32", _I),
                 ("gate_kind", _I), ("gate_w", _P), ("gate_rank", _I), ("gate_z", _P), ("norm_w", _P), ("eps", _F),
                 ("state", _P), ("fresh", _I), ("pos", _P), ("pos0", _L), ("t0", _I), ("n", _I), ("o_buf", _P),
-                ("workspace", _P), ("workspace_bytes", _Z), ("out", _P)]
+                ("workspace", _P), ("workspace_bytes", _Z), ("out", _P),
+                ("rule", _I), ("rate_off", _I), ("rate_bias", _P), ("decay_tanh", _I), ("decay_rate", _F),
+                ("norm_per_head", _I)]
+
+
+class Latent(ctypes.Structure):
+    """socket_latent"""
+    _fields_ = [("dtype", _I), ("B", _I), ("T", _I), ("H", _I), ("dim", _I), ("rot", _I), ("q_rank", _I), ("rank", _I),
+                ("in_", _P), ("in_f32", _I), ("in_stride_b", _L), ("in_stride_t", _L),
+                ("cq_off", _I), ("c_off", _I), ("rot_off", _I), ("q_norm", _P), ("c_norm", _P), ("eps", _F),
+                ("cos_sin", _P), ("n_pos", _L), ("pos0", _L), ("pos", _P),
+                ("cache", _P), ("cache_stride_b", _L), ("cache_stride_t", _L), ("cq_out", _P), ("append", _I),
+                ("q", _P), ("w_uk", _P), ("q_lat", _P)]
+
+
+class LatentAttend(ctypes.Structure):
+    """socket_latent_attention"""
+    _fields_ = [("dtype", _I), ("B", _I), ("T", _I), ("H", _I), ("rank", _I), ("rot", _I), ("vdim", _I),
+                ("q_lat", _P), ("cache", _P), ("cache_stride_b", _L), ("cache_stride_t", _L), ("n_pos", _L), ("pos0", _L),
+                ("pos", _P), ("scale", _F), ("splits", _I), ("o", _P), ("ml", _P),
+                ("w_uv", _P), ("gate", _P), ("gate_f32", _I), ("gate_stride_b", _L), ("gate_stride_t", _L), ("out", _P)]
 
 
 # name -> (restype, argtypes); one entry per declaration in include/socket_hip.h.
@@ -85,15 +114,21 @@ class Recurrence(ctypes.Structure):
 CORE_SIGNATURES = {
     "socket_residual_norm": (_I, [POINTER(Residual), _L, _P]),
     "socket_rows_linear_bf16": (_I, [POINTER(RowsLinear), _P]),
-    "socket_clamped_glu": (_I, [_P, _P, _I, _L, _I, _F, _P]),
+    "socket_gated_unit": (_I, [_P, _P, _I, _L, _I, _I, _F, _P]),
     "socket_rope_half_rows": (_I, [POINTER(RopeHalf), _P]),
     "socket_chunk_ring_store": (_I, [_P, _L, _L, _L, _P, _L, _L, _L, _P, _P, _L, _L, _L, _I, _I, _I, _I, _I, _I, _L, _P]),
     "socket_chunk_attend": (_I, [POINTER(ChunkAttention), _P]),
     "socket_dense_decode_capped_workspace_bytes": (_Z, [_I, _I, _I]),
     "socket_dense_decode_capped": (_I, [_P, _P, _P, _I] + [_L] * 8 + [_P, _P, _L, _L, _P, _Z, _I, _I, _I, _I, _I, _F, _F, _P]),
     "socket_recurrence_step": (_I, [POINTER(Recurrence), _P]),
-    "socket_recurrence_chunk": (_I, [_I]),
-    "socket_recurrence_workspace_bytes": (_Z, [_I, _I, _I, _I, _I]),
+    "socket_recurrence_chunk": (_I, [_I, _I]),
+    "socket_recurrence_workspace_bytes": (_Z, [_I, _I, _I, _I, _I, _I]),
+    "socket_tanh_rows": (_I, [_P, _L, _P, _I, _L, _I, _P]),
+    "socket_latent_rows": (_I, [POINTER(Latent), _P]),
+    "socket_latent_absorb": (_I, [POINTER(Latent), _P]),
+    "socket_rotate_tail": (_I, [_P, _I, _I, _I, _I, _I, _I, _P, _L, _L, _P]),
+    "socket_latent_attend": (_I, [POINTER(LatentAttend), _P]),
+    "socket_latent_values": (_I, [POINTER(LatentAttend), _P]),
     "socket_recurrence_scan": (_I, [POINTER(Recurrence), _P]),
     "socket_recurrence_conv_tail": (_I, [POINTER(Recurrence), _P]),
     "socket_abi_version": (_I, []),
@@ -177,7 +212,7 @@ def _load(path: str, signatures: dict, how: str) -> ctypes.CDLL:
         fn = getattr(handle, name)
         fn.restype = res
         fn.argtypes = args
-    if handle.socket_abi_version() != 4:
+    if handle.socket_abi_version() != 5:
         raise RuntimeError(f"{os.path.basename(path)} ABI version mismatch; rebuild it")
     return handle
 

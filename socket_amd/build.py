@@ -3,8 +3,8 @@
 Run as `python -m socket_amd.build`; `__graft_entry__.build()` calls `build()`.
 Objects are compiled in parallel, one translation unit per kernel family, and
 linked into two libraries next to this file: libsocket_core.so (what every model
-family uses: decode-step helpers, dense attention, chunked attention, gated
-recurrences) and libsocket_hip.so (hashing, scoring, selection and block-sparse
+family uses: decode-step helpers, dense attention, chunked and latent attention,
+gated recurrences) and libsocket_hip.so (hashing, scoring, selection and block-sparse
 attention of the SOCKET path), which depends on it.  `build_core()` makes the first
 alone.
 """
@@ -20,7 +20,8 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB_PATH = os.path.join(HERE, "libsocket_hip.so")
 CORE_PATH = os.path.join(HERE, "libsocket_core.so")
-CORE_SOURCES = ["common.hip", "attend.hip", "decode_ops.hip", "rows.hip", "chunk_attend.hip", "recurrence.hip"]
+CORE_SOURCES = ["common.hip", "attend.hip", "decode_ops.hip", "rows.hip", "chunk_attend.hip", "latent.hip",
+                "recurrence.hip"]
 SOURCES = ["score.hip", "collide.hip", "topk.hip", "hash.hip", "softhash.hip", "block_sparse.hip"]
 ARCH = "gfx950"
 # Packed-FP32 VALU ops are switched off for every device translation unit.
@@ -38,6 +39,7 @@ FILE_FLAGS = {
     "block_sparse.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
     "attend.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],     # the MFMA dense flash-decode, for the same reason
     "chunk_attend.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
+    "latent.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
     "recurrence.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
 }
 

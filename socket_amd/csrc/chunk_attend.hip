@@ -6,7 +6,9 @@
 // position p lives in slot p % chunk, and the visible keys of a decode step are the
 // slots 0 .. p % chunk, a plain prefix.  A prompt portion reads the keys it brings from
 // its own projections and older keys of its first chunk from the ring; the rows of its
-// last chunk are stored into the ring after the attention has read it.
+// last chunk are stored into the ring after the attention has read it.  Full causal attention is
+// the case of one endless chunk; values may be narrower or wider than keys, a second key segment
+// may be shared by all heads, and the output may be gated.
 #include "elem.h"
 
 namespace {
@@ -115,12 +117,12 @@ __device__ __forceinline__ KeySource key_source(const socket_chunk_attention& a,
   s.k_st = a.k_stride_t * es;
   s.v_st = a.v_stride_t * es;
   s.r_ss = a.ring_stride_s * es;
-  s.fresh_from = a.pos ? pos + 1 : a.pos0;       // (a decode step's own key is in the ring already)
+  s.fresh_from = a.pos ? pos + 1 : a.k_from;     // (a decode step's own key is in the ring already)
   s.chunk = a.chunk;
   return s;
 }
 
-// Any head dim up to 512, any type, all arithmetic fp32: one wave per query row.  A block of
+// Any value width up to 512, any type, all arithmetic fp32: one wave per query row.  A block of
 // 64 keys, one key per lane for the scores; for the values a lane owns dims lane, lane + 64, ...
 constexpr int kSimpleWaves = 4;
 constexpr int kSimpleDims = 8;   // dims per lane
@@ -134,12 +136,13 @@ __global__ __launch_bounds__(kSimpleWaves * 64) void chunk_attend_simple_kernel(
   const bool live = r < (int64_t)a.T * a.H;        // (wave-uniform; no barrier below)
   if (!live) return;
   const int t = (int)(r / a.H), h = (int)(r % a.H), g = h / (a.H / a.G);
-  float* qs = ca_lds + wave * (a.D + 64);
-  float* ps = qs + a.D;
+  const int Dq = a.D + a.D2, Dv = a.Dv;
+  float* qs = ca_lds + wave * (Dq + 64);
+  float* ps = qs + Dq;
   const int64_t i = a.pos ? *a.pos : a.pos0 + t;
   const KeySource src = key_source<DT>(a, b, g, i);
   const int64_t q0 = b * a.q_stride_b + t * a.q_stride_t + h * a.q_stride_h;
-  for (int d = lane; d < a.D; d += 64) qs[d] = load_elem<DT>(a.q, q0 + d);
+  for (int d = lane; d < Dq; d += 64) qs[d] = load_elem<DT>(a.q, q0 + d);
   float acc[kSimpleDims];
 #pragma unroll
   for (int e = 0; e < kSimpleDims; ++e) acc[e] = 0.f;
@@ -153,6 +156,8 @@ __global__ __launch_bounds__(kSimpleWaves * 64) void chunk_attend_simple_kernel(
         const char* kp = src.key(j);
         s = 0.f;
         for (int d = 0; d < a.D; ++d) s = fmaf(qs[d], load_elem<DT>(kp, d), s);
+        for (int d = 0; d < a.D2; ++d)
+          s = fmaf(qs[a.D + d], load_elem<DT>(a.k2, b * a.k2_stride_b + j * a.k2_stride_t + d), s);
         s *= a.scale;
         if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
       }
@@ -173,17 +178,20 @@ __global__ __launch_bounds__(kSimpleWaves * 64) void chunk_attend_simple_kernel(
         const char* vp = src.value(j0 + jj);
 #pragma unroll
         for (int e = 0; e < kSimpleDims; ++e)
-          if (lane + 64 * e < a.D) acc[e] = fmaf(pj, load_elem<DT>(vp, lane + 64 * e), acc[e]);
+          if (lane + 64 * e < Dv) acc[e] = fmaf(pj, load_elem<DT>(vp, lane + 64 * e), acc[e]);
       }
       __builtin_amdgcn_wave_barrier();
     }
   }
   l = __shfl(wave_reduce_to_last<false>(l), 63, 64);
   const float inv = l > 0.f ? 1.f / l : 0.f;
-  const int64_t o0 = (((int64_t)b * a.T + t) * a.H + h) * a.D;
+  const int64_t o0 = (((int64_t)b * a.T + t) * a.H + h) * Dv;
+  const int64_t g0 = b * a.gate_stride_b + t * a.gate_stride_t + (int64_t)h * Dv;
 #pragma unroll
-  for (int e = 0; e < kSimpleDims; ++e)
-    if (lane + 64 * e < a.D) store_elem<DT>(a.out, o0 + lane + 64 * e, acc[e] * inv);
+  for (int e = 0; e < kSimpleDims; ++e) {
+    const int d = lane + 64 * e;
+    if (d < Dv) store_elem<DT>(a.out, o0 + d, acc[e] * inv * (a.gate ? sigmoid_f32(load_elem<DT>(a.gate, g0 + d)) : 1.f));
+  }
 }
 
 // ---- bf16 portions on the matrix cores --------------------------------------------------------
@@ -228,17 +236,20 @@ constexpr int kVtPitch = kTileKeys + 8;
 constexpr float kMaxOfflineCap = 60.f;   // exp(60) * 2^31 keys < 3.4e38, exp(-60) > 1.2e-38
 constexpr float kLog2e = 1.4426950408889634f;
 
-template <int DP, int RW, bool ONLINE>
+// DP: key dims (both segments), DVP: value dims, rounded up; SHARED: there is a second segment.
+template <int DP, int DVP, int RW, bool ONLINE, bool SHARED>
 __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_attention a) {
-  constexpr int CH = DP / 8;                 // 16-byte pieces per row
+  constexpr int CH = DP / 8;                 // 16-byte pieces per key
   constexpr int KS = DP / 32;
-  constexpr int DB = DP / 16;
+  constexpr int DB = DVP / 16;
   constexpr int KP = CH + 1;                 // pitch of a K row in pieces (odd: 16 rows hit 16 bank groups)
   constexpr int TASKS = 16 * CH;             // (piece, four keys) per tile
   constexpr int PER = (TASKS + 255) / 256;
+  constexpr int TASKS_V = 16 * (DVP / 8), PER_V = (TASKS_V + 255) / 256;
   constexpr int ROWS = 64 * RW;              // rows per workgroup
   __shared__ __attribute__((aligned(16))) uint4 k_lds[kTileKeys * KP];
-  __shared__ __attribute__((aligned(16))) uint16_t vt_lds[DP * kVtPitch];
+  __shared__ __attribute__((aligned(16))) uint16_t vt_lds[DVP * kVtPitch];
+  const int Dq = SHARED ? a.D + a.D2 : a.D, Dv = a.Dv;
 
   const int Gq = a.H / a.G;
   // kv heads are neighbours in the launch order: with eight of them each XCD's L2 serves one head's
@@ -274,7 +285,7 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
       const int d = (4 * ks + quarter) * 8;
-      qf[w][ks] = (live && d < a.D) ? *reinterpret_cast<const uint4*>(q + d) : make_uint4(0, 0, 0, 0);
+      qf[w][ks] = (live && d < Dq) ? *reinterpret_cast<const uint4*>(q + d) : make_uint4(0, 0, 0, 0);
     }
   }
   ca_f32x4 o[RW][DB];
@@ -289,18 +300,29 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
   const float c1 = a.softcap > 0.f ? 2.f * kLog2e * a.scale / a.softcap : a.scale * kLog2e;
   const float c2 = a.softcap * kLog2e;
 
-  uint4 kr[PER][4], vr[PER][4];
+  uint4 kr[PER][4], vr[PER_V][4];
+  const char* k2 = SHARED ? (const char*)a.k2 + b * a.k2_stride_b * 2 : nullptr;
   auto fetch = [&](int j0) __attribute__((always_inline)) {
 #pragma unroll
     for (int p = 0; p < PER; ++p) {
       const int task = tid + p * 256, piece = task % CH, key0 = 4 * (task / CH);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        kr[p][i] = vr[p][i] = make_uint4(0, 0, 0, 0);
-        if (task < TASKS && piece * 8 < a.D) {
-          const int64_t j = base + min(j0 + key0 + i, end - 1);   // (a live row past the end; masked below)
-          kr[p][i] = *reinterpret_cast<const uint4*>(src.key(j) + piece * 16);
-          vr[p][i] = *reinterpret_cast<const uint4*>(src.value(j) + piece * 16);
+        kr[p][i] = make_uint4(0, 0, 0, 0);
+        if (p < PER_V) vr[p][i] = make_uint4(0, 0, 0, 0);
+        const int64_t j = base + min(j0 + key0 + i, end - 1);   // (a live row past the end; masked below)
+        if (task < TASKS && piece * 8 < Dq) {
+          if (SHARED && piece * 8 >= a.D)
+            kr[p][i] = *reinterpret_cast<const uint4*>(k2 + j * a.k2_stride_t * 2 + (piece * 8 - a.D) * 2);
+          else
+            kr[p][i] = *reinterpret_cast<const uint4*>(src.key(j) + piece * 16);
+        }
+        if (DVP == DP && task < TASKS && piece * 8 < Dv) vr[p][i] = *reinterpret_cast<const uint4*>(src.value(j) + piece * 16);
+        if constexpr (DVP != DP) {
+          const int vpiece = task % (DVP / 8), vkey0 = 4 * (task / (DVP / 8));
+          const int64_t jv = base + min(j0 + vkey0 + i, end - 1);
+          if (p < PER_V && task < TASKS_V && vpiece * 8 < Dv)
+            vr[p][i] = *reinterpret_cast<const uint4*>(src.value(jv) + vpiece * 16);
         }
       }
     }
@@ -308,10 +330,17 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
   auto store = [&]() __attribute__((always_inline)) {
 #pragma unroll
     for (int p = 0; p < PER; ++p) {
-      const int task = tid + p * 256, piece = task % CH, key0 = 4 * (task / CH);
-      if (task >= TASKS) continue;
+      const int task = tid + p * 256;
+      if (task < TASKS) {
+        const int piece = task % CH, key0 = 4 * (task / CH);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) k_lds[(key0 + i) * KP + piece] = kr[p][i];
+        for (int i = 0; i < 4; ++i) k_lds[(key0 + i) * KP + piece] = kr[p][i];
+      }
+    }
+#pragma unroll
+    for (int p = 0; p < PER_V; ++p) {
+      const int task = tid + p * 256, piece = task % (DVP / 8), key0 = 4 * (task / (DVP / 8));
+      if (task >= TASKS_V) continue;
       const uint32_t w[4][4] = {{vr[p][0].x, vr[p][0].y, vr[p][0].z, vr[p][0].w},
                                 {vr[p][1].x, vr[p][1].y, vr[p][1].z, vr[p][1].w},
                                 {vr[p][2].x, vr[p][2].y, vr[p][2].z, vr[p][2].w},
@@ -436,11 +465,18 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
     if (r >= R) continue;
     const float inv = 1.f / sum;
     const int64_t t = r / Gq, h = g * Gq + r % Gq;
-    uint16_t* out = (uint16_t*)a.out + (((int64_t)b * a.T + t) * a.H + h) * a.D;
+    uint16_t* out = (uint16_t*)a.out + (((int64_t)b * a.T + t) * a.H + h) * Dv;
+    const int64_t g0 = b * a.gate_stride_b + t * a.gate_stride_t + h * Dv;
 #pragma unroll
     for (int db = 0; db < DB; ++db) {
       const int d = db * 16 + 4 * quarter;
-      if (d < a.D)
+      if (SHARED && a.gate && d < Dv) {
+        float gate[4];
+        load_vec<DType_bf16, 4>(a.gate, g0 + d, gate);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[w][db][r] *= sigmoid_f32(gate[r]);
+      }
+      if (d < Dv)
         *reinterpret_cast<uint2*>(out + d) = make_uint2(pack_bf16x2(o[w][db][0] * inv, o[w][db][1] * inv),
                                                         pack_bf16x2(o[w][db][2] * inv, o[w][db][3] * inv));
     }
@@ -448,27 +484,34 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
 }
 
 bool mma_fits(const socket_chunk_attention& a) {
-  if (a.force_simple || a.pos || a.dtype != SOCKET_BF16 || a.D % 8 != 0 || a.D > 256) return false;
+  if (a.force_simple || a.pos || a.dtype != SOCKET_BF16 || a.D % 8 != 0 || a.D + a.D2 > 256) return false;
+  if (a.k2 ? a.Dv > 256 || a.softcap > 0.f : a.Dv != a.D || a.gate) return false;
+  if (a.Dv % 8 != 0 || a.D2 % 8 != 0) return false;
   const int64_t strides[] = {a.q_stride_b, a.q_stride_t, a.q_stride_h, a.k_stride_b, a.k_stride_t, a.k_stride_g,
-                             a.v_stride_b, a.v_stride_t, a.v_stride_g, a.ring_stride_b, a.ring_stride_g, a.ring_stride_s};
+                             a.v_stride_b, a.v_stride_t, a.v_stride_g, a.ring_stride_b, a.ring_stride_g, a.ring_stride_s,
+                             a.k2_stride_b, a.k2_stride_t, a.gate_stride_b, a.gate_stride_t};
   for (int64_t st : strides)
     if (st % 8 != 0) return false;
-  const void* ptrs[] = {a.q, a.k_new, a.v_new, a.k_ring, a.v_ring, a.out};
+  const void* ptrs[] = {a.q, a.k_new, a.v_new, a.k_ring, a.v_ring, a.out, a.k2, a.gate};
   for (const void* p : ptrs)
     if (!socket_aligned16(p)) return false;
-  return (int64_t)a.T + a.chunk < (1LL << 30);
+  return a.chunk == INT32_MAX ? a.pos0 + a.T < (1LL << 30) : (int64_t)a.T + a.chunk < (1LL << 30);
 }
 
-template <int DP, int RW>
+template <int DP, int DVP, int RW, bool SHARED>
 int launch_mma(const socket_chunk_attention& a, hipStream_t s) {
   const int64_t rows = (int64_t)a.T * (a.H / a.G);
   const int64_t n = (rows + 64 * RW - 1) / (64 * RW) * a.G * a.B;
   SOCKET_REQUIRE(n < (1LL << 31), SOCKET_ERR_SHAPE);
   const dim3 grid((unsigned)n), block(256);
-  if (a.softcap > 0.f && a.softcap <= kMaxOfflineCap)
-    hipLaunchKernelGGL((chunk_attend_mma_kernel<DP, RW, false>), grid, block, 0, s, a);
-  else
-    hipLaunchKernelGGL((chunk_attend_mma_kernel<DP, RW, true>), grid, block, 0, s, a);
+  if constexpr (!SHARED) {
+    if (a.softcap > 0.f && a.softcap <= kMaxOfflineCap) {
+      hipLaunchKernelGGL((chunk_attend_mma_kernel<DP, DVP, RW, false, false>), grid, block, 0, s, a);
+      SOCKET_LAUNCH_CHECK();
+      return SOCKET_OK;
+    }
+  }
+  hipLaunchKernelGGL((chunk_attend_mma_kernel<DP, DVP, RW, true, SHARED>), grid, block, 0, s, a);
   SOCKET_LAUNCH_CHECK();
   return SOCKET_OK;
 }
@@ -538,26 +581,39 @@ extern "C" int socket_chunk_ring_store(const void* k, int64_t k_sb, int64_t k_st
 }
 
 extern "C" int socket_chunk_attend(const socket_chunk_attention* args, void* stream) {
-  SOCKET_REQUIRE(args && args->q && args->k_ring && args->v_ring && args->out, SOCKET_ERR_NULL);
-  const socket_chunk_attention& a = *args;
+  SOCKET_REQUIRE(args && args->q && args->out, SOCKET_ERR_NULL);
+  socket_chunk_attention a = *args;
+  if (a.Dv == 0) a.Dv = a.D;
+  SOCKET_REQUIRE((a.k_ring && a.v_ring) || (!a.pos && a.k_from == 0), SOCKET_ERR_NULL);
+  SOCKET_REQUIRE(a.pos || (a.k_from >= 0 && a.k_from <= a.pos0), SOCKET_ERR_SHAPE);
+  SOCKET_REQUIRE(a.k2 ? (a.D2 > 0 && !a.pos && a.k_from == 0) : a.D2 == 0, SOCKET_ERR_SHAPE);
+  SOCKET_REQUIRE(a.Dv > 0 && (a.D + a.D2 + 64) * 4 * kSimpleWaves <= 48 * 1024, SOCKET_ERR_UNSUPPORTED);
   SOCKET_REQUIRE(a.pos || (a.k_new && a.v_new), SOCKET_ERR_NULL);
   SOCKET_REQUIRE(a.dtype == SOCKET_F32 || a.dtype == SOCKET_BF16, SOCKET_ERR_UNSUPPORTED);
   SOCKET_REQUIRE(a.B > 0 && a.B <= 65535 && a.T > 0 && a.H > 0 && a.G > 0 && a.H % a.G == 0, SOCKET_ERR_SHAPE);
   SOCKET_REQUIRE(a.chunk > 0 && (!a.pos || a.T == 1) && a.pos0 >= 0, SOCKET_ERR_SHAPE);
-  SOCKET_REQUIRE(a.D > 0 && a.D <= 64 * kSimpleDims, SOCKET_ERR_UNSUPPORTED);
+  SOCKET_REQUIRE(a.D > 0 && a.Dv <= 64 * kSimpleDims, SOCKET_ERR_UNSUPPORTED);
   hipStream_t s = (hipStream_t)stream;
   if (mma_fits(a)) {
-    if (a.D <= 32) return launch_mma<32, 2>(a, s);
-    if (a.D <= 64) return launch_mma<64, 2>(a, s);
-    if (a.D <= 96) return launch_mma<96, 2>(a, s);
-    if (a.D <= 128) return launch_mma<128, 2>(a, s);
-    if (a.D <= 192) return launch_mma<192, 1>(a, s);
-    return launch_mma<256, 1>(a, s);
+    if (a.k2) {
+      const int dq = a.D + a.D2;
+      if (dq <= 64 && a.Dv <= 64) return launch_mma<64, 64, 2, true>(a, s);
+      if (dq <= 96 && a.Dv <= 96) return launch_mma<96, 96, 2, true>(a, s);
+      if (dq <= 128 && a.Dv <= 128) return launch_mma<128, 128, 2, true>(a, s);
+      if (dq <= 192 && a.Dv <= 128) return launch_mma<192, 128, 2, true>(a, s);
+      return launch_mma<256, 256, 1, true>(a, s);
+    }
+    if (a.D <= 32) return launch_mma<32, 32, 2, false>(a, s);
+    if (a.D <= 64) return launch_mma<64, 64, 2, false>(a, s);
+    if (a.D <= 96) return launch_mma<96, 96, 2, false>(a, s);
+    if (a.D <= 128) return launch_mma<128, 128, 2, false>(a, s);
+    if (a.D <= 192) return launch_mma<192, 192, 1, false>(a, s);
+    return launch_mma<256, 256, 1, false>(a, s);
   }
   const int64_t rows = (int64_t)a.T * a.H;
   SOCKET_REQUIRE((rows + kSimpleWaves - 1) / kSimpleWaves < (1LL << 31), SOCKET_ERR_SHAPE);
   const dim3 grid((unsigned)((rows + kSimpleWaves - 1) / kSimpleWaves), (unsigned)a.B), block(kSimpleWaves * 64);
-  const size_t lds = (size_t)kSimpleWaves * (a.D + 64) * 4;
+  const size_t lds = (size_t)kSimpleWaves * (a.D + a.D2 + 64) * 4;
   if (a.dtype == SOCKET_F32) hipLaunchKernelGGL((chunk_attend_simple_kernel<DType_f32>), grid, block, lds, s, a);
   else hipLaunchKernelGGL((chunk_attend_simple_kernel<DType_bf16>), grid, block, lds, s, a);
   SOCKET_LAUNCH_CHECK();

@@ -67,6 +67,15 @@ __device__ __forceinline__ float log1p_f32(float t) {
 }
 __device__ __forceinline__ float softplus_f32(float x) { return fmaxf(x, 0.f) + log1p_f32(exp_f32(-fabsf(x))); }
 
+// 1 - 2 / (e^2x + 1): exact to about one unit of the result's scale 1 (the argument's own scale
+// near 0, where the difference cancels, is served by the odd polynomial's first terms).
+__device__ __forceinline__ float tanh_f32(float x) {
+  const float big = 1.f - 2.f * __builtin_amdgcn_rcpf(exp_f32(2.f * x) + 1.f);
+  const float x2 = x * x;
+  const float small = x * fmaf(x2, fmaf(x2, 2.f / 15.f, -1.f / 3.f), 1.f);
+  return fabsf(x) < 0.05f ? small : big;
+}
+
 // Sum over the workgroup (a multiple of 64 lanes, up to 1024), the same value in every lane.
 // `red` holds one float per wave; two calls in a row need two arrays or a barrier between.
 __device__ __forceinline__ float block_sum(float v, float* red) {

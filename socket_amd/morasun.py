@@ -11,23 +11,17 @@ from typing import Dict, Tuple
 
 import torch
 
+from .checkpoint import only, put
 from .hybrid import BranchSpec, ClampedGLUSpec, HybridArgs, HybridTransformer, LayerSpec
 from .mixers import ChunkAttention, ChunkAttentionSpec, RecurrenceSpec
 
 ARCHITECTURE = "Morasun"
 
 
-def _only(d: dict, keys: str, where: str) -> dict:
-    unknown, missing = set(d) - set(keys.split()), set(keys.split()) - set(d)
-    if unknown or missing:
-        raise ValueError(f"config, {where}: unknown keys {sorted(unknown)}, missing keys {sorted(missing)}")
-    return d
-
-
 def _attention(c: dict, where: str) -> ChunkAttentionSpec:
-    _only(c, "heads kv_heads dim vdim mask rot scale softcap", where)
-    _only(c["mask"], "size", where + ".mask")
-    _only(c["rot"], "base dims", where + ".rot")
+    only(c, "heads kv_heads dim vdim mask rot scale softcap", where)
+    only(c["mask"], "size", where + ".mask")
+    only(c["rot"], "base dims", where + ".rot")
     if c["vdim"] != c["dim"]:
         raise ValueError(f"config, {where}: the values are the keys, so vdim must equal dim")
     return ChunkAttentionSpec(heads=c["heads"], kv_heads=c["kv_heads"], dim=c["dim"], chunk=c["mask"]["size"],
@@ -36,29 +30,29 @@ def _attention(c: dict, where: str) -> ChunkAttentionSpec:
 
 
 def _delta(c: dict, ranks: Tuple[int, int], where: str) -> RecurrenceSpec:
-    _only(c, "heads kv_heads dim vdim conv", where)
+    only(c, "heads kv_heads dim vdim conv", where)
     return RecurrenceSpec(heads=c["heads"], kv_heads=c["kv_heads"], dim=c["dim"], vdim=c["vdim"], decay_rank=ranks[0],
                           delta=True, taps=c["conv"], unit_qk=True, decay="exp_softplus", gate="sigmoid",
                           gate_rank=ranks[1])
 
 
 def _gla(c: dict, rank: int, where: str) -> RecurrenceSpec:
-    _only(c, "heads dim vdim tau", where)
+    only(c, "heads dim vdim tau", where)
     return RecurrenceSpec(heads=c["heads"], kv_heads=c["heads"], dim=c["dim"], vdim=c["vdim"], decay_rank=rank,
                           delta=False, decay="sigmoid_root", tau=float(c["tau"]), gate="silu")
 
 
 def args_from_config(config: dict, shapes: Dict[str, Tuple[int, ...]]) -> HybridArgs:
     """`shapes`: tensor name -> shape, for the inner widths."""
-    _only(config, "architecture layers norm vocab width", "top level")
-    _only(config["norm"], "eps", "norm")
+    only(config, "architecture layers norm vocab width", "top level")
+    only(config["norm"], "eps", "norm")
     layers = []
     for i, lay in enumerate(config["layers"]):
         where, pre = f"layer {i}", f"l{i}.mix"
-        _only(lay, "type mixer mlp", where)
+        only(lay, "type mixer mlp", where)
         c = lay["mixer"]
         if lay["type"] == "parallel":
-            _only(c, "left right left_scale right_scale", where)
+            only(c, "left right left_scale right_scale", where)
             ranks = (shapes[pre + ".right.a1"][0], shapes[pre + ".right.g1"][0])
             branches = [BranchSpec(_attention(c["left"], where + ".left"), float(c["left_scale"]), "left"),
                         BranchSpec(_delta(c["right"], ranks, where + ".right"), float(c["right_scale"]), "right")]
@@ -68,7 +62,7 @@ def args_from_config(config: dict, shapes: Dict[str, Tuple[int, ...]]) -> Hybrid
             raise ValueError(f"config, {where}: unknown layer type {lay['type']!r}")
         mlp = None
         if lay["mlp"] is not None:
-            _only(lay["mlp"], "ff kind limit", where + ".mlp")
+            only(lay["mlp"], "ff kind limit", where + ".mlp")
             if lay["mlp"]["kind"] != "dense":
                 raise ValueError(f"config, {where}: unknown feed-forward kind {lay['mlp']['kind']!r}")
             mlp = ClampedGLUSpec(lay["mlp"]["ff"], float(lay["mlp"]["limit"]))
@@ -77,64 +71,57 @@ def args_from_config(config: dict, shapes: Dict[str, Tuple[int, ...]]) -> Hybrid
                       architecture=ARCHITECTURE)
 
 
-def _put(dst: torch.Tensor, src: torch.Tensor, name: str) -> None:
-    # (vectors kept per head and channel may be stored in either shape)
-    if dst.numel() != src.numel() or (dst.dim() > 1 and tuple(dst.shape) != tuple(src.shape)):
-        raise ValueError(f"tensor {name} has shape {tuple(src.shape)}, expected {tuple(dst.shape)}")
-    dst.copy_(src.reshape(dst.shape))
-
-
 @torch.no_grad()
 def load_tensors(model: HybridTransformer, take, ignore=lambda name: None) -> None:
     """Fill the model's parameters; `take(name)` hands over the checkpoint's tensor of that name,
     `ignore(name)` says that one is not needed."""
-    _put(model.tok_embeddings.weight, take("embed"), "embed")
-    _put(model.norm, take("final.norm"), "final.norm")
-    _put(model.output.weight, take("head"), "head")
+    put(model.tok_embeddings.weight, take("embed"), "embed")
+    put(model.norm, take("final.norm"), "final.norm")
+    put(model.output.weight, take("head"), "head")
     for i, layer in enumerate(model.layers):
         pre = f"l{i}."
         layer.in_proj.zero_()
 
         def rows(tag, name, src):
             at, n = layer.columns.offset[tag + "." + name], layer.columns.rows[tag + "." + name]
-            _put(layer.in_proj[at:at + n], take(src), src)
+            put(layer.in_proj[at:at + n], take(src), src)
 
         for n in ("norm1", "norm1b") + (("norm2", "norm2b") if layer.spec.mlp is not None else ()):
-            _put(getattr(layer, n), take(pre + n), pre + n)
+            put(getattr(layer, n), take(pre + n), pre + n)
         for br, b in zip(layer.branches, layer.spec.branches):
             mix = pre + "mix" + ("." + b.name if b.name else "")
             t, c = br.tag, b.spec
-            _put(br.o, take(mix + ".o"), mix + ".o")
+            put(br.o, take(mix + ".o"), mix + ".o")
             rows(t, "q", mix + ".q")
             rows(t, "k", mix + ".k")
             if isinstance(br, ChunkAttention):
                 continue
             rows(t, "v", mix + ".v")
             rows(t, "a1", mix + ".a1")
-            _put(br.decay_w, take(mix + ".a2"), mix + ".a2")
-            _put(br.norm, take(mix + ".norm"), mix + ".norm")
+            put(br.decay_w, take(mix + ".a2"), mix + ".a2")
+            put(br.norm, take(mix + ".norm"), mix + ".norm")
             if c.delta:
                 rows(t, "b", mix + ".b")
                 rows(t, "g", mix + ".g1")
-                _put(br.gate_w, take(mix + ".g2"), mix + ".g2")
-                _put(br.a_log, take(mix + ".A_log"), mix + ".A_log")
-                _put(br.decay_bias, take(mix + ".dt_bias"), mix + ".dt_bias")
+                put(br.gate_w, take(mix + ".g2"), mix + ".g2")
+                put(br.a_log, take(mix + ".A_log"), mix + ".A_log")
+                put(br.decay_bias, take(mix + ".dt_bias"), mix + ".dt_bias")
             else:
                 rows(t, "g", mix + ".g")
-                _put(br.decay_bias, take(mix + ".a2.b"), mix + ".a2.b")
+                put(br.decay_bias, take(mix + ".a2.b"), mix + ".a2.b")
             if c.delta:
                 at = 0
                 for n in ("q", "k", "v"):
                     w = take(f"{mix}.{n}.conv")
                     if w.shape[1] != c.taps:
                         raise ValueError(f"tensor {mix}.{n}.conv has {w.shape[1]} taps, the config says {c.taps}")
-                    _put(br.conv_w[:, at:at + w.shape[0]], w.t(), f"{mix}.{n}.conv")
+                    put(br.conv_w[:, at:at + w.shape[0]], w.t(), f"{mix}.{n}.conv")
                     at += w.shape[0]
         if layer.spec.mlp is None:
             ignore(pre + "norm2")
             ignore(pre + "norm2b")
         else:
             ff = layer.spec.mlp.ff
-            _put(layer.gate_up[:ff], take(pre + "mlp.gate"), pre + "mlp.gate")
-            _put(layer.gate_up[ff:], take(pre + "mlp.up"), pre + "mlp.up")
-            _put(layer.down, take(pre + "mlp.down"), pre + "mlp.down")
+            put(layer.gate_up[:ff], take(pre + "mlp.gate"), pre + "mlp.gate")
+            put(layer.gate_up[ff:], take(pre + "mlp.up"), pre + "mlp.up")
+            put(layer.down, take(pre + "mlp.down"), pre + "mlp.down")

@@ -13,34 +13,11 @@ from typing import Callable, Dict
 
 import torch
 
-from . import morasun
+from . import guselix, morasun
+from .checkpoint import Checkpoint
 from .hybrid import HybridArgs, HybridTransformer
 from .mixers import GatedRecurrence
 from .model import ModelArgs, Transformer
-
-
-class Checkpoint:
-    """Tensors of a safetensors file, read one at a time; `finish` complains about unread ones."""
-
-    def __init__(self, path: str):
-        from safetensors import safe_open
-        self._file = safe_open(path, framework="pt", device="cpu")
-        self._left = set(self._file.keys())
-        self.shapes = {n: tuple(self._file.get_slice(n).get_shape()) for n in self._left}
-
-    def take(self, name: str) -> torch.Tensor:
-        if name not in self.shapes:
-            raise ValueError(f"the checkpoint has no tensor {name}")
-        self._left.discard(name)
-        return self._file.get_tensor(name)
-
-    def ignore(self, name: str) -> None:
-        """`name` may be in the file and is not needed."""
-        self._left.discard(name)
-
-    def finish(self) -> None:
-        if self._left:
-            raise ValueError(f"the checkpoint has tensors the model does not know: {sorted(self._left)[:8]}")
 
 
 def _load_hybrid(config: dict, ckpt: Checkpoint, device, dtype, design) -> HybridTransformer:
@@ -72,6 +49,7 @@ def _load_llama(config: dict, ckpt: Checkpoint, device, dtype) -> Transformer:
 ARCHITECTURES: Dict[str, Callable] = {
     "Transformer": _load_llama,      # the Llama-style decoder: config.json holds ModelArgs' fields
     morasun.ARCHITECTURE: lambda config, ckpt, device, dtype: _load_hybrid(config, ckpt, device, dtype, morasun),
+    guselix.ARCHITECTURE: lambda config, ckpt, device, dtype: _load_hybrid(config, ckpt, device, dtype, guselix),
 }
 
 
@@ -112,8 +90,11 @@ def random_model(args: HybridArgs, device, dtype=torch.bfloat16, seed: int = 123
         for name, p in m._parameters.items():
             if p is None:
                 continue
-            if name.startswith("norm"):
+            if name.startswith("norm") or name.endswith("norm"):
                 p.fill_(1.0)
+            elif name == "dwa":          # mostly the layer's own result
+                p.fill_(0.25 / max(p.numel() - 1, 1))
+                p[-1] = 0.75
             else:
                 p.normal_(mean=0.0, std=0.02, generator=gen)
         if isinstance(m, GatedRecurrence):

@@ -1,10 +1,11 @@
-"""What a sequence keeps between steps in layers other than full attention.
+"""What a sequence keeps between steps in the layers of mixers.py.
 
+`LatentCache` holds one row per position that all heads of a latent attention share.
 `ChunkRing` holds the keys and values of the chunk a sequence is in: position p in
 row p % chunk, so a decode step's visible keys are the first p % chunk + 1 rows and
 memory does not grow past one chunk.  `RecurrentState` holds a recurrence's fp32
 state and the last inputs of its short convolution.  Both are filled by the kernels
-(csrc/chunk_attend.hip, csrc/recurrence.hip); a portion at position 0 starts them
+(csrc/latent.hip, csrc/chunk_attend.hip, csrc/recurrence.hip); a portion at position 0 starts them
 anew, so a slot can be used again without being cleared.
 """
 from __future__ import annotations
@@ -29,6 +30,24 @@ class ChunkRing:
     def overwritten_by_a_step(self) -> List[Tensor]:
         """Tensors whose old contents a decode step needs again to be repeated: none (a step
         writes its own row and reads it back)."""
+        return []
+
+
+class LatentCache:
+    """Row p: the normed latent of position p, zeros up to a multiple of 8, the rotated key part,
+    zeros up to a multiple of 8."""
+
+    def __init__(self, batch: int, max_seq_length: int, rank: int, rot: int, dtype, device):
+        self.rank, self.rot = rank, rot
+        self.rot_at = (rank + 7) // 8 * 8
+        self.width = self.rot_at + (rot + 7) // 8 * 8
+        self.rows = torch.zeros(batch, max_seq_length, self.width, dtype=dtype, device=device)
+
+    def tensors(self) -> List[Tensor]:
+        return [self.rows]
+
+    def overwritten_by_a_step(self) -> List[Tensor]:
+        """None: a step writes its own row and reads it back."""
         return []
 
 

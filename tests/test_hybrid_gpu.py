@@ -86,7 +86,7 @@ def test_clamped_glu_beyond_its_limits(dev, dtype, ff):
     gu = 4 * _rand(g, 3, 2 * ff)
     t, u = torch.clamp(gu[:, :ff], max=1.5), torch.clamp(gu[:, ff:], -1.5, 1.5)
     assert (gu[:, :ff] > 1.5).any() and (gu[:, :ff] < -4).any() and (gu[:, ff:] < -1.5).any()
-    got = layer_ops.clamped_glu(gu.to(dev, dtype), 1.5).cpu()
+    got = layer_ops.gated_unit(gu.to(dev, dtype), "clamped", 1.5).cpu()
     assert hm.rms_error(got, t * ho.sigmoid(1.702 * t) * (u + 1)) < (1e-6 if dtype == torch.float32 else 4e-3)
 
 
