@@ -29,6 +29,7 @@ CPU oracle timed on the host's cores on a slice of configuration 3.
   python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload c2|c3|c4|c5] [--no-extra]
                   [--only score|score_grouped|select|attend|hash|dense|step|decode|...] [--no-cpu] [--no-parity]
   python bench.py --hybrid all     prefill and decode of the Morasun design beside the Llama-style model
+                                   (--hybrid-design guselix: of the Guselix design beside Morasun)
 """
 from __future__ import annotations
 
@@ -644,15 +645,17 @@ def decode_tok_s(dev, prompt_len, new_tokens, n_layer=None, kinds=("sparse", "de
     return rec
 
 
-def hybrid_bench(dev, size, prompt_len, new_tokens, part="all"):
-    """Prefill and decode throughput of the Morasun design (random weights) beside the Llama-style
-    model of the same width, feed-forward, heads and layers, dense attention: the same prompt
-    length, one sequence, the decode step replayed as a HIP graph."""
+def hybrid_bench(dev, size, prompt_len, new_tokens, part="all", design="morasun"):
+    """Prefill and decode throughput of a design (random weights) beside a model of the same width,
+    feed-forward and layers, dense attention: the Morasun design beside the Llama-style
+    model, the Guselix design beside Morasun.  The same prompt length, one sequence, the decode
+    step replayed as a HIP graph."""
     from socket_amd import generate as gen
-    from socket_amd.workloads import hybrid_args
-    hybrid, llama = hybrid_args(size)
-    rec = {"size": size, "prompt_len": prompt_len, "new_tokens": new_tokens, "batch": 1, "n_layer": llama.n_layer}
-    for name, cfg in (("morasun", hybrid), ("llama", llama)):
+    from socket_amd.workloads import guselix_args, hybrid_args
+    args = (guselix_args if design == "guselix" else hybrid_args)(size)
+    names = ("guselix", "morasun") if design == "guselix" else ("morasun", "llama")
+    rec = {"size": size, "prompt_len": prompt_len, "new_tokens": new_tokens, "batch": 1, "n_layer": args[0].n_layer}
+    for name, cfg in zip(names, args):
         if part not in ("all", name):
             continue
         model = gen.load_random_model(cfg, dev, torch.bfloat16, 1234)
@@ -686,7 +689,9 @@ def main():
     ap.add_argument("--hybrid", default=None, choices=["2k", "4k", "all"],
                     help="instead of the default workload: prefill and decode of the Morasun design at layers of this "
                          "width beside the Llama-style model of the same size")
-    ap.add_argument("--hybrid-part", default="all", choices=["all", "morasun", "llama"])
+    ap.add_argument("--hybrid-design", default="morasun", choices=["morasun", "guselix"],
+                    help="guselix: the Guselix design beside Morasun instead")
+    ap.add_argument("--hybrid-part", default="all", choices=["all", "guselix", "morasun", "llama"])
     ap.add_argument("--prompt-len", type=int, default=8000,
                     help="prompt of --hybrid (the default and --new-tokens end just inside a chunk of 8192)")
     ap.add_argument("--new-tokens", type=int, default=129, help="generated tokens of --hybrid")
@@ -716,7 +721,8 @@ def main():
     torch.cuda.set_device(dev)
     if args.hybrid:
         sizes = ["2k", "4k"] if args.hybrid == "all" else [args.hybrid]
-        print(json.dumps({"hybrid": [hybrid_bench(dev, s, args.prompt_len, args.new_tokens, args.hybrid_part) for s in sizes]}))
+        print(json.dumps({"hybrid": [hybrid_bench(dev, s, args.prompt_len, args.new_tokens, args.hybrid_part,
+                                                  args.hybrid_design) for s in sizes]}))
         return
     if args.only == "block_sparse":
         block_sparse_bench(dev, max(args.steps, 1), args.warmup)

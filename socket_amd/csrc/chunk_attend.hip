@@ -122,10 +122,10 @@ __device__ __forceinline__ KeySource key_source(const socket_chunk_attention& a,
   return s;
 }
 
-// Any value width up to 512, any type, all arithmetic fp32: one wave per query row.  A block of
+// Any value width up to 1024, any type, all arithmetic fp32: one wave per query row.  A block of
 // 64 keys, one key per lane for the scores; for the values a lane owns dims lane, lane + 64, ...
 constexpr int kSimpleWaves = 4;
-constexpr int kSimpleDims = 8;   // dims per lane
+constexpr int kSimpleDims = 16;   // dims per lane
 
 template <class DT>
 __global__ __launch_bounds__(kSimpleWaves * 64) void chunk_attend_simple_kernel(socket_chunk_attention a) {

@@ -445,7 +445,8 @@ def latent_attend(q_lat: Tensor, cache, scale: float, w_uv: Tensor, vdim: int, g
 def tanh_rows(x: Tensor) -> Tensor:
     """tanh of the rows x [B,T,n], a slice of wider rows, as a contiguous tensor."""
     B, T, n = x.shape
-    assert x.stride(2) == 1 and (B == 1 or x.stride(0) == T * x.stride(1))
+    if x.stride(2) != 1 or (B > 1 and x.stride(0) != T * x.stride(1)):
+        x = x.contiguous()
     y = torch.empty(B, T, n, dtype=x.dtype, device=x.device)
     check("socket_tanh_rows", core().socket_tanh_rows(ptr(x), x.stride(1), ptr(y), dtype_enum(x.dtype), B * T, n,
                                                       stream_ptr(x.device)))

@@ -173,3 +173,20 @@ def hybrid_args(size: str):
     llama = ModelArgs(block_size=131072, vocab_size=vocab, n_layer=n, n_head=heads, n_local_heads=kv, dim=width,
                       intermediate_size=ff, rope_base=500000)
     return HybridArgs(vocab_size=vocab, dim=width, layers=layers, architecture="Morasun"), llama
+
+
+def guselix_args(size: str):
+    """Guselix geometries with a real model's layer sizes, and the Morasun geometry of the same width,
+    feed-forward and number of layers: (HybridArgs, HybridArgs)."""
+    from .guselix import general_delta
+    from .hybrid import BranchSpec, HybridArgs, LayerSpec, SiluGLUSpec
+    from .mixers import LatentAttentionSpec
+    other, _ = hybrid_args(size)
+    width, ff, heads, q_rank = {"2k": (2048, 8192, 16, 768), "4k": (4096, 14336, 32, 1536)}[size]
+    mlp = SiluGLUSpec(ff, bias=True)
+    delta = general_delta(width // 64, 64, 128)
+    latent = LatentAttentionSpec(heads=heads, dim=128, rot_dim=64, vdim=128, q_rank=q_rank, kv_rank=512, rot_base=500000.0,
+                                 scale=192 ** -0.5)
+    layers = [LayerSpec([BranchSpec(delta if i % 2 == 0 else latent)], mlp) for i in range(other.n_layer)]
+    return HybridArgs(vocab_size=other.vocab_size, dim=width, layers=layers, architecture="Guselix", embed_scale=float(width) ** 0.5,
+                      tied_head=True, post_norm=False, depth_average=True), other

@@ -39,7 +39,7 @@ CONFIGS = {
                      latent_layer(latent(2, 40, 16, 8, 24, 72, 90.0, 0.21)), delta_layer(delta(1, 64), mlp(24)), latent_layer()]),
     # nothing is a multiple of eight (scalar paths), a value width above the key's, one head
     "odd": config([delta_layer(delta(2, 10), mlp(21)), latent_layer(latent(5, 9, 6, 19, 13, 11, 33.0, 0.4), mlp(33)),
-                   latent_layer(latent(1, 1, 2, 1, 1, 1, 3.0, 1.0)), delta_layer(delta(3, 7))], width=37, vocab=53, scale=1.0),
+                   latent_layer(latent(1, 3, 2, 1, 5, 7, 3.0, 1.0)), delta_layer(delta(3, 7))], width=37, vocab=53, scale=1.0),
     # wider heads (32-token chunks of the recurrence, other sizes of the matrix-core kernels), more heads than a tile
     "wide": config([delta_layer(delta(1, 136)), latent_layer(latent(18, 96, 32, 64, 64, 136, 2000.0), mlp(72)),
                     delta_layer(delta(2, 80), mlp(64)), latent_layer(latent(2, 128, 64, 128, 128, 320, 9000.0))], width=64, vocab=120,
