@@ -202,7 +202,7 @@ __global__ __launch_bounds__(kSimpleWaves * 64) void chunk_attend_simple_kernel(
 // N index: lane x holds row x % 16 in every accumulator):
 //   S^T[key, row] = K . Q^T,   O^T[dim, row] = V^T . P^T
 // so the weights a lane computes are the operand it has to supply.  V is transposed on its way
-// into LDS: rows of 72 elements, the sixteen 4-key groups of a row at group ^ (dim / 8 % 16).
+// into LDS: rows of NK + 8 elements, the 4-key groups of a row at group ^ (dim / 8 % (NK / 4)).
 // Weights are computed in fp32 and enter the second product as a sum of two bf16 numbers.
 //
 // With a soft cap the scores are bounded by it, and exp(score) needs no running maximum
@@ -231,23 +231,23 @@ __device__ __forceinline__ uint32_t pack_bf16x2(float lo, float hi) {
   return r.u;
 }
 
-constexpr int kTileKeys = 64;
-constexpr int kVtPitch = kTileKeys + 8;
 constexpr float kMaxOfflineCap = 60.f;   // exp(60) * 2^31 keys < 3.4e38, exp(-60) > 1.2e-38
 constexpr float kLog2e = 1.4426950408889634f;
 
 // DP: key dims (both segments), DVP: value dims, rounded up; SHARED: there is a second segment.
-template <int DP, int DVP, int RW, bool ONLINE, bool SHARED>
-__global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_attention a) {
+// NK: keys of a tile (32 where 64 would leave one wave per SIMD).
+template <int DP, int DVP, int RW, int NK, bool ONLINE, bool SHARED>
+__global__ __launch_bounds__(256, NK == 32 ? 2 : 1) void chunk_attend_mma_kernel(socket_chunk_attention a) {
   constexpr int CH = DP / 8;                 // 16-byte pieces per key
   constexpr int KS = DP / 32;
   constexpr int DB = DVP / 16;
   constexpr int KP = CH + 1;                 // pitch of a K row in pieces (odd: 16 rows hit 16 bank groups)
-  constexpr int TASKS = 16 * CH;             // (piece, four keys) per tile
+  constexpr int kVtPitch = NK + 8, GROUPS = NK / 4, NB = NK / 16;
+  constexpr int TASKS = GROUPS * CH;             // (piece, four keys) per tile
   constexpr int PER = (TASKS + 255) / 256;
-  constexpr int TASKS_V = 16 * (DVP / 8), PER_V = (TASKS_V + 255) / 256;
+  constexpr int TASKS_V = GROUPS * (DVP / 8), PER_V = (TASKS_V + 255) / 256;
   constexpr int ROWS = 64 * RW;              // rows per workgroup
-  __shared__ __attribute__((aligned(16))) uint4 k_lds[kTileKeys * KP];
+  __shared__ __attribute__((aligned(16))) uint4 k_lds[NK * KP];
   __shared__ __attribute__((aligned(16))) uint16_t vt_lds[DVP * kVtPitch];
   const int Dq = SHARED ? a.D + a.D2 : a.D, Dv = a.Dv;
 
@@ -351,29 +351,29 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
         uint2 t;
         t.x = __builtin_amdgcn_perm(w[1][e >> 1], w[0][e >> 1], sel);
         t.y = __builtin_amdgcn_perm(w[3][e >> 1], w[2][e >> 1], sel);
-        *reinterpret_cast<uint2*>(vt_lds + (piece * 8 + e) * kVtPitch + (((key0 >> 2) ^ (piece & 15)) << 2)) = t;
+        *reinterpret_cast<uint2*>(vt_lds + (piece * 8 + e) * kVtPitch + (((key0 >> 2) ^ (piece & (GROUPS - 1))) << 2)) = t;
       }
     }
   };
 
   fetch(0);
-  for (int j0 = 0; j0 < end; j0 += kTileKeys) {
+  for (int j0 = 0; j0 < end; j0 += NK) {
     __syncthreads();   // the previous tile has been consumed
     store();
     __syncthreads();
-    if (j0 + kTileKeys < end) fetch(j0 + kTileKeys);
-    if (!wave_live || j0 > iw1 || j0 + kTileKeys - 1 < cw0) continue;   // (wave-uniform)
-    const bool open = j0 + kTileKeys - 1 <= iw0 && j0 >= cw1;
+    if (j0 + NK < end) fetch(j0 + NK);
+    if (!wave_live || j0 > iw1 || j0 + NK - 1 < cw0) continue;   // (wave-uniform)
+    const bool open = j0 + NK - 1 <= iw0 && j0 >= cw1;
 
-    ca_f32x4 s[RW][4];
+    ca_f32x4 s[RW][NB];
 #pragma unroll
     for (int w = 0; w < RW; ++w)
 #pragma unroll
-      for (int nb = 0; nb < 4; ++nb) s[w][nb] = ca_f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int nb = 0; nb < NB; ++nb) s[w][nb] = ca_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
-      for (int nb = 0; nb < 4; ++nb) {
+      for (int nb = 0; nb < NB; ++nb) {
         const uint4 kf = k_lds[(nb * 16 + prow) * KP + 4 * ks + quarter];
 #pragma unroll
         for (int w = 0; w < RW; ++w) s[w][nb] = mfma_bf16(kf, qf[w][ks], s[w][nb]);
@@ -385,7 +385,7 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
       if constexpr (ONLINE) {
         float mb = -INFINITY;
 #pragma unroll
-        for (int nb = 0; nb < 4; ++nb)
+        for (int nb = 0; nb < NB; ++nb)
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const int j = j0 + nb * 16 + 4 * quarter + r;
@@ -411,7 +411,7 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
         }
       }
 #pragma unroll
-      for (int nb = 0; nb < 4; ++nb)
+      for (int nb = 0; nb < NB; ++nb)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           float p;
@@ -428,7 +428,7 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
         }
     }
 #pragma unroll
-    for (int c = 0; c < 2; ++c) {
+    for (int c = 0; c < NB / 2; ++c) {
       uint4 ph[RW], pl[RW];   // slots 0..3: keys 32c + 4q + r, slots 4..7: keys 32c + 16 + 4q + r
 #pragma unroll
       for (int w = 0; w < RW; ++w) {
@@ -444,7 +444,7 @@ __global__ __launch_bounds__(256) void chunk_attend_mma_kernel(socket_chunk_atte
 #pragma unroll
       for (int db = 0; db < DB; ++db) {
         const uint16_t* vrow = vt_lds + (db * 16 + prow) * kVtPitch;
-        const int swz = (2 * db + (prow >> 3)) & 15;
+        const int swz = (2 * db + (prow >> 3)) & (GROUPS - 1);
         const uint2 lo = *reinterpret_cast<const uint2*>(vrow + (((8 * c + quarter) ^ swz) << 2));
         const uint2 hi = *reinterpret_cast<const uint2*>(vrow + (((8 * c + 4 + quarter) ^ swz) << 2));
         const uint4 vf = make_uint4(lo.x, lo.y, hi.x, hi.y);
@@ -498,7 +498,7 @@ bool mma_fits(const socket_chunk_attention& a) {
   return a.chunk == INT32_MAX ? a.pos0 + a.T < (1LL << 30) : (int64_t)a.T + a.chunk < (1LL << 30);
 }
 
-template <int DP, int DVP, int RW, bool SHARED>
+template <int DP, int DVP, int RW, bool SHARED, int NK = 64>
 int launch_mma(const socket_chunk_attention& a, hipStream_t s) {
   const int64_t rows = (int64_t)a.T * (a.H / a.G);
   const int64_t n = (rows + 64 * RW - 1) / (64 * RW) * a.G * a.B;
@@ -506,12 +506,12 @@ int launch_mma(const socket_chunk_attention& a, hipStream_t s) {
   const dim3 grid((unsigned)n), block(256);
   if constexpr (!SHARED) {
     if (a.softcap > 0.f && a.softcap <= kMaxOfflineCap) {
-      hipLaunchKernelGGL((chunk_attend_mma_kernel<DP, DVP, RW, false, false>), grid, block, 0, s, a);
+      hipLaunchKernelGGL((chunk_attend_mma_kernel<DP, DVP, RW, NK, false, false>), grid, block, 0, s, a);
       SOCKET_LAUNCH_CHECK();
       return SOCKET_OK;
     }
   }
-  hipLaunchKernelGGL((chunk_attend_mma_kernel<DP, DVP, RW, true, SHARED>), grid, block, 0, s, a);
+  hipLaunchKernelGGL((chunk_attend_mma_kernel<DP, DVP, RW, NK, true, SHARED>), grid, block, 0, s, a);
   SOCKET_LAUNCH_CHECK();
   return SOCKET_OK;
 }
@@ -599,9 +599,9 @@ extern "C" int socket_chunk_attend(const socket_chunk_attention* args, void* str
       const int dq = a.D + a.D2;
       if (dq <= 64 && a.Dv <= 64) return launch_mma<64, 64, 2, true>(a, s);
       if (dq <= 96 && a.Dv <= 96) return launch_mma<96, 96, 2, true>(a, s);
-      if (dq <= 128 && a.Dv <= 128) return launch_mma<128, 128, 2, true>(a, s);
-      if (dq <= 192 && a.Dv <= 128) return launch_mma<192, 128, 2, true>(a, s);
-      return launch_mma<256, 256, 1, true>(a, s);
+      if (dq <= 128 && a.Dv <= 128) return launch_mma<128, 128, 2, true, 32>(a, s);
+      if (dq <= 192 && a.Dv <= 128) return launch_mma<192, 128, 2, true, 32>(a, s);
+      return launch_mma<256, 256, 1, true, 32>(a, s);
     }
     if (a.D <= 32) return launch_mma<32, 32, 2, false>(a, s);
     if (a.D <= 64) return launch_mma<64, 64, 2, false>(a, s);

@@ -22,67 +22,116 @@ constexpr float kLatLog2e = 1.4426950408889634f;
 int round8(int n) { return (n + 7) & ~7; }
 __device__ __forceinline__ int round8d(int n) { return (n + 7) & ~7; }
 
-__device__ __forceinline__ float load_in(const socket_latent& a, int64_t i) {
-  return a.in_f32 ? ((const float*)a.in)[i] : bf16_bits_to_f32(((const uint16_t*)a.in)[i]);
+// V neighbouring elements of a projected row.
+template <int V>
+__device__ __forceinline__ void load_in(const socket_latent& a, int64_t i, float* out) {
+  if (a.in_f32) load_vec<DType_f32, V>(a.in, i, out);
+  else load_vec<DType_bf16, V>(a.in, i, out);
 }
 
-// The cache row of token (b, t), by the whole workgroup.
-template <class DT>
-__device__ __forceinline__ void cache_row(const socket_latent& a, int b, int t, float* red) {
+// Element i of a rotate-half of `rot` elements at position p: x(k) gives the element before.
+template <class X>
+__device__ __forceinline__ float rotated(const float* cos_sin, int64_t p, int rot, int i, X x) {
+  const int half = rot / 2, pair = i < half ? i : i - half;
+  const float2 f = *reinterpret_cast<const float2*>(cos_sin + (p * half + pair) * 2);
+  const float u = x(pair), v = x(pair + half);
+  return i < half ? fmaf(u, f.x, -(v * f.y)) : fmaf(v, f.x, u * f.y);
+}
+
+// The cache row of token (b, t) and, with QUERY, its normed query latent, by a workgroup of N lanes.
+template <class DT, int V, bool QUERY, int N>
+__device__ __forceinline__ void project_row(const socket_latent& a, int b, int t, float (*red)[4]) {
   const int64_t p = a.pos ? *a.pos : a.pos0 + t;
-  if (p < 0 || p >= a.n_pos) return;                    // (uniform)
+  const bool ok = p >= 0 && p < a.n_pos;                // (uniform)
   const int64_t row = b * a.in_stride_b + t * a.in_stride_t;
-  const int64_t dst = b * a.cache_stride_b + p * a.cache_stride_t;
-  float ss = 0.f;
-  for (int i = threadIdx.x; i < a.rank; i += kLatThreads) {
-    const float x = load_in(a, row + a.c_off + i);
-    ss = fmaf(x, x, ss);
+  const int64_t dst = b * a.cache_stride_b + p * a.cache_stride_t, cq = ((int64_t)b * a.T + t) * a.q_rank;
+  float sc = 0.f, sq = 0.f;
+  for (int i = threadIdx.x * V; i < a.rank; i += N * V) {
+    float x[V];
+    load_in<V>(a, row + a.c_off + i, x);
+#pragma unroll
+    for (int e = 0; e < V; ++e) sc = fmaf(x[e], x[e], sc);
   }
-  const float rs = rsqrt_f32(block_sum(ss, red) / (float)a.rank + a.eps);
-  const int rank_p = round8d(a.rank), rot_p = round8d(a.rot), half = a.rot / 2;
-  for (int i = threadIdx.x; i < rank_p; i += kLatThreads)
-    store_elem<DT>(a.cache, dst + i, i < a.rank ? load_in(a, row + a.c_off + i) * rs * a.c_norm[i] : 0.f);
-  for (int i = threadIdx.x; i < rot_p; i += kLatThreads) {
-    float y = 0.f;
-    if (i < a.rot) {
-      const int pair = i < half ? i : i - half;
-      const float u = load_in(a, row + a.rot_off + pair), v = load_in(a, row + a.rot_off + pair + half);
-      const float2 f = *reinterpret_cast<const float2*>(a.cos_sin + (p * half + pair) * 2);
-      y = i < half ? fmaf(u, f.x, -(v * f.y)) : fmaf(v, f.x, u * f.y);
+  if constexpr (QUERY) {
+    for (int i = threadIdx.x * V; i < a.q_rank; i += N * V) {
+      float x[V];
+      load_in<V>(a, row + a.cq_off + i, x);
+#pragma unroll
+      for (int e = 0; e < V; ++e) sq = fmaf(x[e], x[e], sq);
     }
+  }
+  const float rc = rsqrt_f32(block_sum(sc, red[0]) / (float)a.rank + a.eps);
+  if constexpr (QUERY) {
+    const float rq = rsqrt_f32(block_sum(sq, red[1]) / (float)a.q_rank + a.eps);
+    for (int i = threadIdx.x * V; i < a.q_rank; i += N * V) {
+      float x[V], w[V];
+      load_in<V>(a, row + a.cq_off + i, x);
+      load_vec<DType_f32, V>(a.q_norm, i, w);
+#pragma unroll
+      for (int e = 0; e < V; ++e) x[e] = x[e] * rq * w[e];
+      store_vec<DT, V>(a.cq_out, cq + i, x);
+    }
+  }
+  if (!ok) return;
+  const int rank_p = round8d(a.rank), rot_p = round8d(a.rot);
+  for (int i = threadIdx.x * V; i < rank_p; i += N * V) {
+    float x[V], w[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) x[e] = w[e] = 0.f;
+    if (i < a.rank) {
+      load_in<V>(a, row + a.c_off + i, x);
+      load_vec<DType_f32, V>(a.c_norm, i, w);
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) x[e] = x[e] * rc * w[e];
+    store_vec<DT, V>(a.cache, dst + i, x);
+  }
+  for (int i = N - 1 - threadIdx.x; i < rot_p; i += N) {          // (the lanes with the least to do so far)
+    const float y = i < a.rot ? rotated(a.cos_sin, p, a.rot, i, [&](int k) {
+      float x;
+      load_in<1>(a, row + a.rot_off + k, &x);
+      return x;
+    }) : 0.f;
     store_elem<DT>(a.cache, dst + rank_p + i, y);
   }
 }
 
-template <class DT>
+template <class DT, int V>
 __global__ __launch_bounds__(kLatThreads) void latent_rows_kernel(socket_latent a) {
   __shared__ float red[2][4];
-  const int t = blockIdx.x, b = blockIdx.y;
-  if (a.cq_out) {
-    const int64_t src = b * a.in_stride_b + t * a.in_stride_t + a.cq_off, dst = ((int64_t)b * a.T + t) * a.q_rank;
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < a.q_rank; i += kLatThreads) {
-      const float x = load_in(a, src + i);
-      ss = fmaf(x, x, ss);
-    }
-    const float rs = rsqrt_f32(block_sum(ss, red[0]) / (float)a.q_rank + a.eps);
-    for (int i = threadIdx.x; i < a.q_rank; i += kLatThreads) store_elem<DT>(a.cq_out, dst + i, load_in(a, src + i) * rs * a.q_norm[i]);
-  }
-  cache_row<DT>(a, b, t, red[1]);
+  if (a.cq_out) project_row<DT, V, true, kLatThreads>(a, blockIdx.y, blockIdx.x, red);
+  else project_row<DT, V, false, kLatThreads>(a, blockIdx.y, blockIdx.x, red);
 }
 
-template <class DT>
+// V pairs per lane.
+template <class DT, int V>
 __global__ __launch_bounds__(256) void rotate_tail_kernel(void* q, int T, int H, int dim, int rot, const float* cos_sin,
                                                           int64_t pos0, int64_t items) {
   const int64_t w = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (w >= items) return;
-  const int half = rot / 2, pair = (int)(w % half);
-  const int64_t head = w / half, t = head / H % T;
+  const int half = rot / 2, units = half / V;
+  const int64_t head = w / units, t = head / H % T;
+  const int pair = (int)(w % units) * V;
   const int64_t at = head * (dim + rot) + dim + pair;
-  const float u = load_elem<DT>(q, at), v = load_elem<DT>(q, at + half);
-  const float2 f = *reinterpret_cast<const float2*>(cos_sin + ((pos0 + t) * half + pair) * 2);
-  store_elem<DT>(q, at, fmaf(u, f.x, -(v * f.y)));
-  store_elem<DT>(q, at + half, fmaf(v, f.x, u * f.y));
+  float u[V], v[V], f[2 * V];
+  load_vec<DT, V>(q, at, u);
+  load_vec<DT, V>(q, at + half, v);
+  const float* cs = cos_sin + ((pos0 + t) * half + pair) * 2;
+  if constexpr (V == 8) {
+    load_vec<DType_f32, 8>(cs, 0, f);
+    load_vec<DType_f32, 8>(cs, 8, f + 8);
+  } else {
+    f[0] = cs[0];
+    f[1] = cs[1];
+  }
+#pragma unroll
+  for (int e = 0; e < V; ++e) {
+    const float x = fmaf(u[e], f[2 * e], -(v[e] * f[2 * e + 1])), y = fmaf(v[e], f[2 * e], u[e] * f[2 * e + 1]);
+    u[e] = x;
+    v[e] = y;
+  }
+  store_vec<DT, V>(q, at, u);
+  store_vec<DT, V>(q, at + half, v);
 }
 
 // ---- query side of a step ---------------------------------------------------------------------
@@ -94,7 +143,7 @@ constexpr int kAbsCols = 64, kAbsGroups = kLatThreads / 8, kAbsRows = 4;
 template <class DT, bool VEC>
 __global__ __launch_bounds__(kLatThreads) void latent_absorb_kernel(socket_latent a) {
   __shared__ __attribute__((aligned(16))) float part[kAbsGroups][kAbsCols + 4];
-  __shared__ float red[4];
+  __shared__ float red[2][4];
   const int tid = threadIdx.x, h = blockIdx.y, b = blockIdx.z / a.T, t = blockIdx.z % a.T;
   const int rank_p = round8d(a.rank), rot_p = round8d(a.rot), width = rank_p + rot_p;
   const float* q = a.q + ((int64_t)blockIdx.z * a.H + h) * (a.dim + a.rot);
@@ -102,18 +151,10 @@ __global__ __launch_bounds__(kLatThreads) void latent_absorb_kernel(socket_laten
   if (blockIdx.x == gridDim.x - 1) {
     const int64_t p0 = a.pos ? *a.pos : a.pos0 + t;
     const int64_t p = p0 < 0 ? 0 : (p0 >= a.n_pos ? a.n_pos - 1 : p0);
-    const int half = a.rot / 2;
-    for (int i = tid; i < rot_p; i += kLatThreads) {
-      float y = 0.f;
-      if (i < a.rot) {
-        const int pair = i < half ? i : i - half;
-        const float u = q[a.dim + pair], v = q[a.dim + pair + half];
-        const float2 f = *reinterpret_cast<const float2*>(a.cos_sin + (p * half + pair) * 2);
-        y = i < half ? fmaf(u, f.x, -(v * f.y)) : fmaf(v, f.x, u * f.y);
-      }
-      store_elem<DT>(a.q_lat, dst + rank_p + i, y);
-    }
-    if (a.append && h == 0) cache_row<DT>(a, b, t, red);
+    for (int i = tid; i < rot_p; i += kLatThreads)
+      store_elem<DT>(a.q_lat, dst + rank_p + i,
+                     i < a.rot ? rotated(a.cos_sin, p, a.rot, i, [&](int k) { return q[a.dim + k]; }) : 0.f);
+    if (a.append && h == 0) project_row<DT, 1, false, kLatThreads>(a, b, t, red);
     return;
   }
   const int c0 = blockIdx.x * kAbsCols, lane8 = tid & 7, grp = tid >> 3, c = c0 + lane8 * 8;
@@ -158,18 +199,19 @@ __global__ __launch_bounds__(kLatThreads) void latent_absorb_kernel(socket_laten
 
 // ---- attention over the cache rows ------------------------------------------------------------
 //
-// A wave takes 16 keys at a time (tiles dealt round the launch's waves) and 16 heads, and keeps its
-// own running maximum; nothing is shared until the end.  Keys go from memory straight into
-// the registers that are the first product's operand, S^T[key, head] = K Q^T (16x16x32), and from
-// there into the wave's own LDS rows, of which the second, O^T[dim, head] = V^T P^T (16x16x16),
-// needs columns: a lane reads 8 neighbouring dims of four keys and so feeds eight accumulators,
-// accumulator i holding dims 8 m + i of a block of 128.  The weights a lane computes are the
-// operand it has to supply; they enter as a sum of two bf16 numbers.
+// A workgroup takes tiles of 64 keys (dealt round the launch's workgroups) for 16 RT heads; the
+// next tile's rows are in registers while a tile in LDS is worked on.  A wave has one 16-key
+// subtile and 16 heads of the first product, S^T[key, head] = K Q^T; the waves agree on the
+// tile's maxima and hand the weights on through LDS, each as a sum of two bf16 numbers; in the
+// second, O^T[dim, head] = V^T P^T, a wave has 64 dims and every head and key.  That product's key
+// rows are the columns of the LDS tile: a lane reads 4 neighbouring dims of eight keys and so feeds
+// four accumulators, accumulator i holding dims 4 m + i of the wave's block.  The keys of a 32-key
+// step are in the order the weights come in: slots 0 .. 3 are keys 4 quarter + r of the first
+// subtile, slots 4 .. 7 those of the second.
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 la_bf16x8;
-typedef __attribute__((__vector_size__(4 * sizeof(short)))) short la_s16x4;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float la_f32x4;
 
-__device__ __forceinline__ la_f32x4 mfma_k32(const uint4& x, const uint4& y, la_f32x4 c) {
+__device__ __forceinline__ la_f32x4 mfma_bf16(const uint4& x, const uint4& y, la_f32x4 c) {
   union {
     uint4 u;
     la_bf16x8 v;
@@ -178,186 +220,213 @@ __device__ __forceinline__ la_f32x4 mfma_k32(const uint4& x, const uint4& y, la_
   b.u = y;
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, c, 0, 0, 0);
 }
-__device__ __forceinline__ la_f32x4 mfma_k16(const uint2& x, const uint2& y, la_f32x4 c) {
-  union {
-    uint2 u;
-    la_s16x4 v;
-  } a, b;
-  a.u = x;
-  b.u = y;
-  return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(a.v, b.v, c, 0, 0, 0);
-}
 __device__ __forceinline__ uint32_t pack2(float lo, float hi) {
-  return (uint32_t)f32_to_bf16_bits(lo) | ((uint32_t)f32_to_bf16_bits(hi) << 16);
+  typedef __bf16 bf2 __attribute__((ext_vector_type(2)));
+  typedef float f2 __attribute__((ext_vector_type(2)));
+  union {
+    bf2 v;
+    uint32_t u;
+  } r;
+  r.v = __builtin_convertvector(f2{lo, hi}, bf2);
+  return r.u;
 }
-__device__ __forceinline__ void wave_lds_fence() {
-  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-  __builtin_amdgcn_wave_barrier();
-  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-}
 
-constexpr int kAttWaves = 4;
+constexpr int kAttThreads = 512, kAttWaves = kAttThreads / 64;
+constexpr int kAttKeys = 64, kAttSub = kAttKeys / 16;
+constexpr int kAttBlock = 64;             // dims of a wave in the second product
 
-template <int KS>
-constexpr int att_pitch() { return KS * 32 + 8; }      // elements of an LDS row
-
-template <int KS, int NV>
-__global__ __launch_bounds__(kAttWaves * 64, 1) void latent_attend_kernel(socket_latent_attention a) {
-  constexpr int PITCH = att_pitch<KS>();
-  static_assert(KS * 32 >= NV * 128, "values are a prefix of the keys");
-  extern __shared__ __attribute__((aligned(16))) uint16_t la_lds[];
-  __shared__ float sm[kAttWaves][16], sl[kAttWaves][16];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+// KS: key dims in steps of 32; RT: heads in tiles of 16.
+template <int KS, int RT>
+__global__ __launch_bounds__(kAttThreads, 1) void latent_attend_kernel(socket_latent_attention a) {
+  constexpr int PITCH = KS * 32 + 16;     // elements of an LDS row (four rows are half the banks apart)
+  constexpr int PIECES = KS * 4, PER = kAttKeys * PIECES / kAttThreads;
+  static_assert(KS % 2 == 0 && kAttKeys * PIECES % kAttThreads == 0 && RT * kAttSub <= kAttWaves, "work does not deal out");
+  extern __shared__ __attribute__((aligned(16))) uint16_t la_lds[];        // kAttKeys x PITCH
+  __shared__ uint2 ph[RT][kAttSub][64], pl[RT][kAttSub][64];
+  __shared__ float top[RT][kAttSub][16], shrink[RT][16], sums[RT][kAttSub][16];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int x16 = lane & 15, quarter = lane >> 4;
-  const int split = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z / a.T, t = blockIdx.z % a.T;
+  const int split = blockIdx.x, h0 = blockIdx.y * 16 * RT, b = blockIdx.z / a.T, t = blockIdx.z % a.T;
   const int rank_p = round8d(a.rank), width = rank_p + round8d(a.rot);
-  const int64_t p = (a.pos ? *a.pos : a.pos0) + t;
-  const int len = (int)(p < 0 ? 0 : (p >= a.n_pos ? a.n_pos : p + 1));
-  const int n_tiles = (len + 15) / 16, stride = a.splits * kAttWaves;
-  uint16_t* mine = la_lds + wave * 16 * PITCH;
+  const uint16_t* rows = (const uint16_t*)a.cache + b * a.cache_stride_b;
 
-  uint4 qf[KS], kr[KS];
-  const bool head_ok = h0 + x16 < a.H;
-  const uint16_t* q = (const uint16_t*)a.q_lat + ((int64_t)blockIdx.z * a.H + (head_ok ? h0 + x16 : 0)) * width;
-#pragma unroll
-  for (int ks = 0; ks < KS; ++ks) {
-    const int d = (4 * ks + quarter) * 8;
-    qf[ks] = head_ok && d < width ? *reinterpret_cast<const uint4*>(q + d) : make_uint4(0, 0, 0, 0);
-  }
+  // (the first rows are requested before the position is known: rows that are not visible become zero
+  // on their way into LDS)
+  uint4 kr[PER];
   auto fetch = [&](int tile) __attribute__((always_inline)) {
-    const int j = min(tile * 16 + x16, len - 1);
-    const uint16_t* row = (const uint16_t*)a.cache + b * a.cache_stride_b + j * a.cache_stride_t;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int at = tid + i * kAttThreads, piece = at % PIECES;
+      const int64_t j = min((int64_t)tile * kAttKeys + at / PIECES, a.n_pos - 1);
+      kr[i] = piece * 8 < width ? *reinterpret_cast<const uint4*>(rows + j * a.cache_stride_t + piece * 8) : make_uint4(0, 0, 0, 0);
+    }
+  };
+  fetch(split);
+  const int rt = wave / kAttSub, sub = wave % kAttSub;
+  const bool scores = rt < RT;
+  uint4 qf[KS];
+  {
+    const int h = h0 + rt * 16 + x16;
+    const bool live = scores && h < a.H;
+    const uint16_t* q = (const uint16_t*)a.q_lat + ((int64_t)blockIdx.z * a.H + (live ? h : 0)) * width;
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
       const int d = (4 * ks + quarter) * 8;
-      kr[ks] = d < width ? *reinterpret_cast<const uint4*>(row + d) : make_uint4(0, 0, 0, 0);
+      qf[ks] = live && d < width ? *reinterpret_cast<const uint4*>(q + d) : make_uint4(0, 0, 0, 0);
     }
-  };
-  la_f32x4 o[NV * 8];
+  }
+  const int64_t p = (a.pos ? *a.pos : a.pos0) + t;
+  const int len = (int)(p < 0 ? 0 : (p >= a.n_pos ? a.n_pos : p + 1));
+  const int n_tiles = (len + kAttKeys - 1) / kAttKeys;
+
+  la_f32x4 o[RT][4];
 #pragma unroll
-  for (int i = 0; i < NV * 8; ++i) o[i] = la_f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int r = 0; r < RT; ++r)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[r][i] = la_f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
   const float c1 = a.scale * kLatLog2e;
-  int tile = split * kAttWaves + wave;
-  if (tile < n_tiles) fetch(tile);
-  for (; tile < n_tiles; tile += stride) {
-    la_f32x4 s = {0.f, 0.f, 0.f, 0.f};
+  const int d0 = wave * kAttBlock;
+  const bool values = d0 < rank_p;
+  for (int tile = split; tile < n_tiles; tile += a.splits) {
+    __syncthreads();                                    // the previous tile has been consumed
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      s = mfma_k32(kr[ks], qf[ks], s);
-      *reinterpret_cast<uint4*>(mine + x16 * PITCH + (4 * ks + quarter) * 8) = kr[ks];
-    }
-    if (tile + stride < n_tiles) fetch(tile + stride);
-    float mb = -INFINITY;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int j = tile * 16 + 4 * quarter + r;
-      s[r] = j < len ? s[r] * c1 : -INFINITY;
-      mb = fmaxf(mb, s[r]);
-    }
-    mb = fmaxf(mb, lane_xor16(mb));
-    mb = fmaxf(mb, lane_xor32(mb));                     // (finite: a tile has a visible key)
-    const float mn = fmaxf(m, mb), alpha = __builtin_amdgcn_exp2f(m - mn);
-    m = mn;
-    l *= alpha;
-    if (__builtin_amdgcn_ballot_w64(alpha != 1.f) != 0) {
-#pragma unroll
-      for (int i = 0; i < NV * 8; ++i)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) o[i][r] *= alpha;
-    }
-    float w[4];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      w[r] = __builtin_amdgcn_exp2f(s[r] - mn);
-      l += w[r];
-    }
-    const uint2 ph = make_uint2(pack2(w[0], w[1]), pack2(w[2], w[3]));
-    const uint2 pl = make_uint2(pack2(w[0] - __uint_as_float(ph.x << 16), w[1] - __uint_as_float(ph.x & 0xffff0000u)),
-                                pack2(w[2] - __uint_as_float(ph.y << 16), w[3] - __uint_as_float(ph.y & 0xffff0000u)));
-    wave_lds_fence();
-#pragma unroll
-    for (int nv = 0; nv < NV; ++nv) {
-      uint4 v[4];
-#pragma unroll
-      for (int j = 0; j < 4; ++j) v[j] = *reinterpret_cast<const uint4*>(mine + (4 * quarter + j) * PITCH + nv * 128 + x16 * 8);
-#pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const uint32_t sel = (i & 1) ? 0x07060302u : 0x05040100u;
-        const uint2 f = make_uint2(__builtin_amdgcn_perm((&v[1].x)[i >> 1], (&v[0].x)[i >> 1], sel),
-                                   __builtin_amdgcn_perm((&v[3].x)[i >> 1], (&v[2].x)[i >> 1], sel));
-        o[nv * 8 + i] = mfma_k16(f, ph, o[nv * 8 + i]);
-        o[nv * 8 + i] = mfma_k16(f, pl, o[nv * 8 + i]);
-      }
-    }
-    wave_lds_fence();                                   // (the rows are rewritten by the next tile)
-  }
-
-  // ---- the workgroup's waves together
-  l += lane_xor16(l);
-  l += lane_xor32(l);
-  if (quarter == 0) {
-    sm[wave][x16] = m;
-    sl[wave][x16] = l;
-  }
-  __syncthreads();
-  float top = -INFINITY, sum = 0.f;
-#pragma unroll
-  for (int w = 0; w < kAttWaves; ++w) top = fmaxf(top, sm[w][x16]);
-  const bool none = top == -INFINITY;
-  if (!none)
-#pragma unroll
-    for (int w = 0; w < kAttWaves; ++w) sum += sl[w][x16] * __builtin_amdgcn_exp2f(sm[w][x16] - top);
-  const float f = none ? 0.f : __builtin_amdgcn_exp2f(m - top);
-  float* acc = reinterpret_cast<float*>(la_lds);        // [16][rank_p]
-  for (int w = 0; w < kAttWaves; ++w) {
-    if (wave == w) {
-#pragma unroll
-      for (int nv = 0; nv < NV; ++nv)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int d = nv * 128 + 8 * (4 * quarter + r);
-          if (d < rank_p) {
-            float* at = acc + x16 * rank_p + d;
-            float4 lo = make_float4(o[nv * 8][r] * f, o[nv * 8 + 1][r] * f, o[nv * 8 + 2][r] * f, o[nv * 8 + 3][r] * f);
-            float4 hi = make_float4(o[nv * 8 + 4][r] * f, o[nv * 8 + 5][r] * f, o[nv * 8 + 6][r] * f, o[nv * 8 + 7][r] * f);
-            if (w > 0) {
-              const float4 pl = *reinterpret_cast<const float4*>(at), ph = *reinterpret_cast<const float4*>(at + 4);
-              lo = make_float4(lo.x + pl.x, lo.y + pl.y, lo.z + pl.z, lo.w + pl.w);
-              hi = make_float4(hi.x + ph.x, hi.y + ph.y, hi.z + ph.z, hi.w + ph.w);
-            }
-            *reinterpret_cast<float4*>(at) = lo;
-            *reinterpret_cast<float4*>(at + 4) = hi;
-          }
-        }
+    for (int i = 0; i < PER; ++i) {
+      const int at = tid + i * kAttThreads, key = at / PIECES;
+      const bool seen = tile * kAttKeys + key < len;
+      *reinterpret_cast<uint4*>(la_lds + key * PITCH + at % PIECES * 8) = seen ? kr[i] : make_uint4(0, 0, 0, 0);
     }
     __syncthreads();
+    if (tile + a.splits < n_tiles) fetch(tile + a.splits);
+    la_f32x4 s = {0.f, 0.f, 0.f, 0.f};
+    if (scores) {
+      const uint16_t* k = la_lds + (16 * sub + x16) * PITCH + quarter * 8;
+      la_f32x4 s1 = {0.f, 0.f, 0.f, 0.f};                // (two sums: neighbouring products do not wait for each other)
+#pragma unroll
+      for (int ks = 0; ks < KS; ks += 2) {
+        s = mfma_bf16(*reinterpret_cast<const uint4*>(k + ks * 32), qf[ks], s);
+        s1 = mfma_bf16(*reinterpret_cast<const uint4*>(k + ks * 32 + 32), qf[ks + 1], s1);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) s[r] += s1[r];
+      float mb = -INFINITY;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        s[r] = tile * kAttKeys + 16 * sub + 4 * quarter + r < len ? s[r] * c1 : -INFINITY;
+        mb = fmaxf(mb, s[r]);
+      }
+      mb = fmaxf(mb, lane_xor16(mb));
+      mb = fmaxf(mb, lane_xor32(mb));
+      if (quarter == 0) top[rt][sub][x16] = mb;
+    }
+    __syncthreads();
+    if (scores) {
+      float mn = m;
+#pragma unroll
+      for (int i = 0; i < kAttSub; ++i) mn = fmaxf(mn, top[rt][i][x16]);   // (finite: a tile has a visible key)
+      const float alpha = __builtin_amdgcn_exp2f(m - mn);
+      m = mn;
+      l *= alpha;
+      float w[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        w[r] = __builtin_amdgcn_exp2f(s[r] - mn);
+        l += w[r];
+      }
+      const uint2 hi = make_uint2(pack2(w[0], w[1]), pack2(w[2], w[3]));
+      ph[rt][sub][lane] = hi;
+      pl[rt][sub][lane] = make_uint2(pack2(w[0] - __uint_as_float(hi.x << 16), w[1] - __uint_as_float(hi.x & 0xffff0000u)),
+                                     pack2(w[2] - __uint_as_float(hi.y << 16), w[3] - __uint_as_float(hi.y & 0xffff0000u)));
+      if (sub == 0 && quarter == 0) shrink[rt][x16] = alpha;
+    }
+    __syncthreads();
+    if (values) {                                       // (wave-uniform)
+#pragma unroll
+      for (int r = 0; r < RT; ++r) {
+        const float alpha = shrink[r][x16];
+        if (__builtin_amdgcn_ballot_w64(alpha != 1.f) != 0) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[r][i][e] *= alpha;
+        }
+      }
+#pragma unroll
+      for (int c = 0; c < kAttSub / 2; ++c) {
+        uint2 v[8];
+#pragma unroll
+        for (int k = 0; k < 8; ++k)
+          v[k] = *reinterpret_cast<const uint2*>(la_lds + (32 * c + 16 * (k >> 2) + 4 * quarter + (k & 3)) * PITCH + d0 + x16 * 4);
+        uint4 hi[RT], lo[RT];
+#pragma unroll
+        for (int r = 0; r < RT; ++r) {
+          const uint2 h0_ = ph[r][2 * c][lane], h1 = ph[r][2 * c + 1][lane], l0 = pl[r][2 * c][lane], l1 = pl[r][2 * c + 1][lane];
+          hi[r] = make_uint4(h0_.x, h0_.y, h1.x, h1.y);
+          lo[r] = make_uint4(l0.x, l0.y, l1.x, l1.y);
+        }
+        uint4 f[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const uint32_t sel = (i & 1) ? 0x07060302u : 0x05040100u;
+          uint32_t w[4];
+#pragma unroll
+          for (int k = 0; k < 4; ++k)
+            w[k] = __builtin_amdgcn_perm(i < 2 ? v[2 * k + 1].x : v[2 * k + 1].y, i < 2 ? v[2 * k].x : v[2 * k].y, sel);
+          f[i] = make_uint4(w[0], w[1], w[2], w[3]);
+#pragma unroll
+          for (int r = 0; r < RT; ++r) o[r][i] = mfma_bf16(f[i], hi[r], o[r][i]);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int r = 0; r < RT; ++r) o[r][i] = mfma_bf16(f[i], lo[r], o[r][i]);
+      }
+    }
   }
+
   const int64_t part = ((int64_t)blockIdx.z * a.splits + split) * a.H + h0;
-  const int heads = min(16, a.H - h0);
-  for (int i = threadIdx.x * 4; i < heads * rank_p; i += kAttWaves * 256)
-    *reinterpret_cast<float4*>(a.o + part * rank_p + i) = *reinterpret_cast<const float4*>(acc + i);
-  if (wave == 0 && quarter == 0 && head_ok) {
-    a.ml[(part + x16) * 2] = top;
-    a.ml[(part + x16) * 2 + 1] = sum;
+  if (values && split < n_tiles) {
+#pragma unroll
+    for (int r = 0; r < RT; ++r)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int d = d0 + 4 * (4 * quarter + e), h = r * 16 + x16;
+        if (h0 + h < a.H && d < rank_p)
+          *reinterpret_cast<float4*>(a.o + (part + h) * rank_p + d) = make_float4(o[r][0][e], o[r][1][e], o[r][2][e], o[r][3][e]);
+      }
+  }
+  if (scores) {
+    l += lane_xor16(l);
+    l += lane_xor32(l);
+    if (quarter == 0) sums[rt][sub][x16] = l;
+  }
+  __syncthreads();
+  if (scores && sub == 0 && quarter == 0 && h0 + rt * 16 + x16 < a.H) {
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < kAttSub; ++i) sum += sums[rt][i][x16];
+    *reinterpret_cast<float2*>(a.ml + (part + rt * 16 + x16) * 2) = make_float2(m, sum);
   }
 }
 
 // ---- value side of a step -----------------------------------------------------------------------
 //
-// Grid (rows of w_uv in slices of 16, heads, tokens).  The first weights are requested before the
-// partial results are merged.
+// Grid (rows of w_uv in slices of 64, heads, tokens).  The first weights are requested before the
+// partial results are merged, which eight groups of lanes share.
+constexpr int kValThreads = 1024, kValWaves = kValThreads / 64;
 constexpr int kValRows = 4;               // per wave
+constexpr int kValGroups = 8, kValLanes = kValThreads / kValGroups;
 constexpr int kMaxSplits = 256;
+constexpr int kMaxMerge = 4 * kValLanes;  // widest row whose merge the groups share
 
 template <class DT, bool VEC>
-__global__ __launch_bounds__(kLatThreads) void latent_values_kernel(socket_latent_attention a) {
-  extern __shared__ __attribute__((aligned(16))) float lv_lds[];   // rank_p
-  __shared__ float share[kMaxSplits];
+__global__ __launch_bounds__(kValThreads) void latent_values_kernel(socket_latent_attention a) {
+  extern __shared__ __attribute__((aligned(16))) float lv_lds[];   // rank_p, then kValGroups x rank_p
+  __shared__ float share[kMaxSplits], red[kValWaves], red2[kValWaves];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int h = blockIdx.y, b = blockIdx.z / a.T, t = blockIdx.z % a.T;
   const int rank_p = round8d(a.rank);
-  const int d0 = (blockIdx.x * (kLatThreads / 64) + wave) * kValRows;
+  const int d0 = (blockIdx.x * kValWaves + wave) * kValRows;
   const int64_t w0 = ((int64_t)h * a.vdim + d0) * a.rank;
   float w[kValRows][8];
   auto request = [&](int c) __attribute__((always_inline)) {
@@ -383,32 +452,48 @@ __global__ __launch_bounds__(kLatThreads) void latent_values_kernel(socket_laten
     gate = a.gate_f32 ? ((const float*)a.gate)[g0 + d0 + lane] : load_elem<DT>(a.gate, g0 + d0 + lane);
   const int64_t part = (int64_t)blockIdx.z * a.splits * a.H + h;
   if (a.ml) {
-    // (a.splits <= 256: a lane per split)
-    __shared__ float red[4], red2[4];
-    const float m = tid < a.splits ? a.ml[(part + (int64_t)tid * a.H) * 2] : -INFINITY;
-    const float l = tid < a.splits ? a.ml[(part + (int64_t)tid * a.H) * 2 + 1] : 0.f;
-    const float mw = wave_reduce_to_last<true>(m);
+    float2 ml = make_float2(-INFINITY, 0.f);           // (a lane per split: at most 256)
+    if (tid < a.splits) ml = *reinterpret_cast<const float2*>(a.ml + (part + (int64_t)tid * a.H) * 2);
+    const float mw = wave_reduce_to_last<true>(ml.x);
     if (lane == 63) red[wave] = mw;
     __syncthreads();
     const float top = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
-    const float f = m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m - top);
-    const float total = block_sum(l * f, red2);
+    const float f = ml.x == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(ml.x - top);
+    const float total = block_sum(ml.y * f, red2);
     if (tid < a.splits) share[tid] = total > 0.f ? f / total : 0.f;
     __syncthreads();
   } else {
     if (tid == 0) share[0] = 1.f;
     __syncthreads();
   }
-  for (int c = tid * 2; c < rank_p; c += kLatThreads * 2) {
-    float2 s = make_float2(0.f, 0.f);
+  if (a.splits > 1 && rank_p <= kMaxMerge) {
+    const int grp = tid / kValLanes, c = tid % kValLanes * 4;
+    float* mine = lv_lds + (1 + grp) * rank_p;
+    if (c < rank_p) {
+      float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
 #pragma unroll 8
-    for (int k = 0; k < a.splits; ++k) {
-      const float2 v = *reinterpret_cast<const float2*>(a.o + (part + (int64_t)k * a.H) * rank_p + c);
-      const float f = share[k];
-      s.x = f > 0.f ? fmaf(f, v.x, s.x) : s.x;          // (an empty split's values are not read into the sum)
-      s.y = f > 0.f ? fmaf(f, v.y, s.y) : s.y;
+      for (int k = grp; k < a.splits; k += kValGroups) {
+        const float f = share[k];                       // (0: the split saw nothing and wrote nothing)
+        float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (f > 0.f) v = *reinterpret_cast<const float4*>(a.o + (part + (int64_t)k * a.H) * rank_p + c);
+        s = make_float4(fmaf(f, v.x, s.x), fmaf(f, v.y, s.y), fmaf(f, v.z, s.z), fmaf(f, v.w, s.w));
+      }
+      *reinterpret_cast<float4*>(mine + c) = s;
     }
-    *reinterpret_cast<float2*>(lv_lds + c) = s;
+    __syncthreads();
+    if (tid < rank_p) {
+      float s = 0.f;
+#pragma unroll
+      for (int g = 0; g < kValGroups; ++g) s += lv_lds[(1 + g) * rank_p + tid];
+      lv_lds[tid] = s;
+    }
+  } else {
+    for (int c = tid; c < rank_p; c += kValThreads) {
+      float s = 0.f;
+      for (int k = 0; k < a.splits; ++k)
+        if (share[k] > 0.f) s = fmaf(share[k], a.o[(part + (int64_t)k * a.H) * rank_p + c], s);
+      lv_lds[c] = s;
+    }
   }
   __syncthreads();
   float acc[kValRows];
@@ -448,19 +533,24 @@ int check_latent(const socket_latent* p) {
   return SOCKET_OK;
 }
 
-template <int KS, int NV>
+template <int KS, int RT>
 int launch_attend(const socket_latent_attention& a, hipStream_t s) {
-  auto kern = latent_attend_kernel<KS, NV>;
-  size_t lds = (size_t)kAttWaves * 16 * att_pitch<KS>() * 2;
-  const size_t merge = (size_t)16 * round8(a.rank) * 4;
-  if (merge > lds) lds = merge;
-  if (lds > 48 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
+  auto kern = latent_attend_kernel<KS, RT>;
+  const size_t lds = (size_t)kAttKeys * (KS * 32 + 16) * 2;
+  if (lds > 32 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
                                              hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
     return SOCKET_ERR_LAUNCH;
-  hipLaunchKernelGGL(kern, dim3((unsigned)a.splits, (unsigned)((a.H + 15) / 16), (unsigned)(a.B * a.T)),
-                     dim3(kAttWaves * 64), lds, s, a);
+  hipLaunchKernelGGL(kern, dim3((unsigned)a.splits, (unsigned)((a.H + 16 * RT - 1) / (16 * RT)), (unsigned)(a.B * a.T)),
+                     dim3(kAttThreads), lds, s, a);
   SOCKET_LAUNCH_CHECK();
   return SOCKET_OK;
+}
+
+template <int KS>
+int launch_attend_heads(const socket_latent_attention& a, hipStream_t s) {
+  // (two tiles of heads per workgroup once there are more workgroups than CUs; neighbours share the L2 before)
+  const int64_t wgs = (int64_t)a.splits * ((a.H + 15) / 16) * a.B * a.T;
+  return a.H <= 16 || wgs <= socket_device_limits().cu_count ? launch_attend<KS, 1>(a, s) : launch_attend<KS, 2>(a, s);
 }
 
 }  // namespace
@@ -473,8 +563,17 @@ extern "C" int socket_latent_rows(const socket_latent* args, void* stream) {
   SOCKET_REQUIRE(!a.cq_out || a.q_rank > 0, SOCKET_ERR_SHAPE);
   const dim3 grid((unsigned)a.T, (unsigned)a.B), block(kLatThreads);
   hipStream_t s = (hipStream_t)stream;
-  if (a.dtype == SOCKET_F32) hipLaunchKernelGGL((latent_rows_kernel<DType_f32>), grid, block, 0, s, a);
-  else hipLaunchKernelGGL((latent_rows_kernel<DType_bf16>), grid, block, 0, s, a);
+  const bool vec = a.rank % 8 == 0 && a.c_off % 8 == 0 && a.in_stride_b % 8 == 0 && a.in_stride_t % 8 == 0 &&
+                   a.cache_stride_b % 8 == 0 && a.cache_stride_t % 8 == 0 && socket_aligned16(a.in) && socket_aligned16(a.cache) &&
+                   socket_aligned16(a.c_norm) &&
+                   (!a.cq_out || (a.q_rank % 8 == 0 && a.cq_off % 8 == 0 && socket_aligned16(a.cq_out) && socket_aligned16(a.q_norm)));
+  if (a.dtype == SOCKET_F32) {
+    if (vec) hipLaunchKernelGGL((latent_rows_kernel<DType_f32, 8>), grid, block, 0, s, a);
+    else hipLaunchKernelGGL((latent_rows_kernel<DType_f32, 1>), grid, block, 0, s, a);
+  } else {
+    if (vec) hipLaunchKernelGGL((latent_rows_kernel<DType_bf16, 8>), grid, block, 0, s, a);
+    else hipLaunchKernelGGL((latent_rows_kernel<DType_bf16, 1>), grid, block, 0, s, a);
+  }
   SOCKET_LAUNCH_CHECK();
   return SOCKET_OK;
 }
@@ -485,12 +584,20 @@ extern "C" int socket_rotate_tail(void* q, int dtype, int B, int T, int H, int d
   SOCKET_REQUIRE(dtype == SOCKET_F32 || dtype == SOCKET_BF16, SOCKET_ERR_UNSUPPORTED);
   SOCKET_REQUIRE(B > 0 && T > 0 && H > 0 && dim >= 0 && rot > 0 && rot % 2 == 0, SOCKET_ERR_SHAPE);
   SOCKET_REQUIRE(pos0 >= 0 && pos0 + T <= n_pos, SOCKET_ERR_SHAPE);
-  const int64_t items = (int64_t)B * T * H * (rot / 2);
+  const bool v8 = dim % 8 == 0 && rot % 16 == 0 && socket_aligned16(q) && socket_aligned16(cos_sin);
+  const int64_t items = (int64_t)B * T * H * (rot / 2) / (v8 ? 8 : 1);
   SOCKET_REQUIRE((items + 255) / 256 < (1LL << 31), SOCKET_ERR_SHAPE);
   const dim3 grid((unsigned)((items + 255) / 256)), block(256);
   hipStream_t s = (hipStream_t)stream;
-  if (dtype == SOCKET_F32) hipLaunchKernelGGL((rotate_tail_kernel<DType_f32>), grid, block, 0, s, q, T, H, dim, rot, cos_sin, pos0, items);
-  else hipLaunchKernelGGL((rotate_tail_kernel<DType_bf16>), grid, block, 0, s, q, T, H, dim, rot, cos_sin, pos0, items);
+#define SOCKET_ROT(DT, V) hipLaunchKernelGGL((rotate_tail_kernel<DT, V>), grid, block, 0, s, q, T, H, dim, rot, cos_sin, pos0, items)
+  if (dtype == SOCKET_F32) {
+    if (v8) SOCKET_ROT(DType_f32, 8);
+    else SOCKET_ROT(DType_f32, 1);
+  } else {
+    if (v8) SOCKET_ROT(DType_bf16, 8);
+    else SOCKET_ROT(DType_bf16, 1);
+  }
+#undef SOCKET_ROT
   SOCKET_LAUNCH_CHECK();
   return SOCKET_OK;
 }
@@ -526,11 +633,12 @@ extern "C" int socket_latent_attend(const socket_latent_attention* args, void* s
                  socket_aligned16(a.q_lat) && socket_aligned16(a.o), SOCKET_ERR_ALIGN);
   const int rank_p = round8(a.rank), width = rank_p + round8(a.rot);
   hipStream_t s = (hipStream_t)stream;
-  if (rank_p <= 128 && width <= 128) return launch_attend<4, 1>(a, s);
-  if (rank_p <= 128 && width <= 192) return launch_attend<6, 1>(a, s);
-  if (rank_p <= 256 && width <= 320) return launch_attend<10, 2>(a, s);
-  if (rank_p <= 512 && width <= 576) return launch_attend<18, 4>(a, s);
-  if (rank_p <= 512 && width <= 640) return launch_attend<20, 4>(a, s);
+  SOCKET_REQUIRE(rank_p <= kAttWaves * kAttBlock, SOCKET_ERR_UNSUPPORTED);
+  if (width <= 128) return launch_attend_heads<4>(a, s);
+  if (width <= 192) return launch_attend_heads<6>(a, s);
+  if (width <= 320) return launch_attend_heads<10>(a, s);
+  if (width <= 576) return launch_attend_heads<18>(a, s);
+  if (width <= 640) return launch_attend_heads<20>(a, s);
   return SOCKET_ERR_UNSUPPORTED;
 }
 
@@ -542,9 +650,9 @@ extern "C" int socket_latent_values(const socket_latent_attention* args, void* s
   SOCKET_REQUIRE((int64_t)a.B * a.T <= 65535 && a.splits >= 1 && a.splits <= kMaxSplits && (a.ml || a.splits == 1), SOCKET_ERR_SHAPE);
   const int rank_p = round8(a.rank);
   SOCKET_REQUIRE((size_t)rank_p * 4 <= 40 * 1024, SOCKET_ERR_UNSUPPORTED);
-  const int per_wg = kLatThreads / 64 * kValRows;
-  const dim3 grid((unsigned)((a.vdim + per_wg - 1) / per_wg), (unsigned)a.H, (unsigned)(a.B * a.T)), block(kLatThreads);
-  const size_t lds = (size_t)rank_p * 4;
+  const int per_wg = kValWaves * kValRows;
+  const dim3 grid((unsigned)((a.vdim + per_wg - 1) / per_wg), (unsigned)a.H, (unsigned)(a.B * a.T)), block(kValThreads);
+  const size_t lds = (size_t)rank_p * 4 * (rank_p <= kMaxMerge ? 1 + kValGroups : 1);
   hipStream_t s = (hipStream_t)stream;
   const bool vec = a.rank % 8 == 0 && socket_aligned16(a.w_uv);
   if (a.dtype == SOCKET_F32) {

@@ -391,9 +391,10 @@ def latent_absorb(q: Tensor, w_uk: Tensor, cache, cos_sin: Tensor, *, pos0: int 
 
 
 def latent_splits(capacity: int, tokens: int, heads: int) -> int:
-    """Workgroups that share a token's keys: a few 16-key tiles per wave, about one workgroup per CU."""
-    groups = tokens * ((heads + 15) // 16)
-    return max(1, min(64, 256 // groups, (capacity + 127) // 128))
+    """Workgroups that share a token's keys: a tile of 64 keys each, from 128 tiles on at least two, and
+    about one workgroup per CU at most."""
+    tiles = (capacity + 63) // 64
+    return max(1, min(256 // (tokens * ((heads + 15) // 16)), tiles if tiles <= 128 else max(128, tiles // 2)))
 
 
 @torch.no_grad()

@@ -199,7 +199,7 @@ def test_latent_cache_layout_and_splits():
         for tokens in (1, 5, 300):
             for heads in (1, 16, 130):
                 n = latent_splits(cap, tokens, heads)
-                assert 1 <= n <= 64 and (n == 1 or n * tokens * ((heads + 15) // 16) <= 256)
+                assert 1 <= n <= 256 and (n == 1 or n * tokens * ((heads + 15) // 16) <= 256)
 
 
 def test_rows_of_a_slice_are_evenly_spaced():
